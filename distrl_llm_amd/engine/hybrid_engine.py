@@ -103,6 +103,8 @@ class HybridEngine:
         self.model = model
         self.cfg = cfg
         self.spec = model.spec
+        if self.spec.norm_center and self.spec.block != "hyper":
+            raise ValueError("the layer norm is available in the hyper block only")
         self.device = device if device is not None else model.device
         self.dtype = model.dtype_
         self._seq_counter = 0
@@ -411,9 +413,10 @@ class HybridEngine:
 
     def _mix_window_attention(self, i, m, L, hm, meta, proj=None, x32=None):
         """Windowed softmax attention. Biases come with the projection GEMM;
-        q/k norm, rotation, the fold of the score-mixing matrix into the
-        queries and the page write are one kernel; distance bias, window,
-        softmax and output gate are the attention kernel's."""
+        short convolution, q/k norm, rotation, query temperature, the fold of
+        the score-mixing matrix into the queries and the page write are one
+        kernel; distance bias, window, softmax, the difference of two maps
+        and the output gate are the attention kernel's."""
         if proj is None:
             proj = F.linear(hm, L.in_w, L.in_b if m.qkv_bias else None)
         cache = self.pool.unit_rows(i, m)
@@ -426,19 +429,24 @@ class HybridEngine:
             proj, m.heads, m.kv_heads, m.dim, m.vdim,
             L.q_norm_w if m.qk_norm else None, L.k_norm_w if m.qk_norm else None,
             self.spec.norm_eps, meta["positions"], freqs, mag,
-            L.talk if m.score_mix else None, meta["page_slot"], cache)
+            L.talk if m.score_mix else None, meta["page_slot"], cache,
+            m.maps, m.qk_unit, m.q_temp,
+            ((L.conv_w, self.slots.mixer_tails[i], meta["cu"], meta["tok_seq"],
+              meta["slots"]) if m.conv_taps else None))
         gate = None
-        if m.out_gate:
-            g0 = m.q_size + m.k_size + m.v_size
-            gate = proj[:, g0:g0 + m.heads]
+        if m.gate_size:
+            g0 = m.conv_channels
+            gate = proj[:, g0:g0 + m.gate_size]
         o = SM.window_attention(
             q, cache, m.heads, m.kv_heads, m.dim, m.vdim, m.score_mix,
             meta["block_tables"], self.pool.block_size, meta["cu"],
             meta["tok_seq"], meta["positions"], m.scale, m.window,
             m.keep_first, L.dist_r1 if m.log_distance else None,
             L.dist_r2 if m.log_distance else None, gate, self.dtype,
-            tiles=meta["wide_tiles"], max_tile=meta["max_wide_tile"])
-        return F.linear(o, L.out_w)
+            tiles=meta["wide_tiles"], max_tile=meta["max_wide_tile"],
+            maps=m.maps, lam_w=L.lam_w if m.maps == 2 else None, diff=m.diff,
+            eps=self.spec.norm_eps)
+        return F.linear(o, L.out_w, L.out_b if m.out_bias else None)
 
     def _mix_delta(self, i, m, L, hm, meta, proj=None, x32=None):
         if proj is None:
@@ -501,7 +509,9 @@ class HybridEngine:
     def _ff(self, f, L, hb):
         if isinstance(f, GluSpec):
             gu = F.linear(hb, L.gu_w)
-            act = SM.silu_glu(gu) if f.act == "silu" else SM.capped_glu(gu, f.limit)
+            act = (SM.silu_glu(gu) if f.act == "silu"
+                   else SM.gelu_glu(gu) if f.act == "gelu_tanh"
+                   else SM.capped_glu(gu, f.limit))
             return F.linear(act, L.down_w), None
         if isinstance(f, MlpSpec):
             return F.linear(SM.gelu_tanh(F.linear(hb, L.up_w)), L.down_w), None
@@ -532,15 +542,34 @@ class HybridEngine:
             x = self._layers_post_norm(tokens, meta, capture)
         elif S.block == "pre_norm":
             x = self._layers_pre_norm(tokens, meta, capture)
+        elif S.block == "hyper":
+            x = self._layers_hyper(tokens, meta, capture)
         else:
             x = self._layers_parallel_gated(tokens, meta, capture)
         if want_rows.numel() == 0:
             return torch.empty(0, S.vocab_size, dtype=torch.float32,
                                device=x.device)
-        _, hb = SM.offset_rmsnorm(x[want_rows], M.final_norm_w, S.norm_eps, dt,
-                                  S.norm_offset, S.norm_groups)
-        logits = F.linear(hb, M.head).float()
+        if S.block == "hyper":
+            hb = SM.hyper_close_norm(x, want_rows, M.final_norm_w, S.norm_eps, dt,
+                                     S.norm_center)
+        else:
+            _, hb = SM.offset_rmsnorm(x[want_rows], M.final_norm_w, S.norm_eps, dt,
+                                      S.norm_offset, S.norm_groups)
+        logits = F.linear(hb, M.head)
+        if S.logit_softcap:
+            return SM.cap_logits(logits, S.logit_scale, S.logit_softcap)
+        logits = logits.float()
         return logits * S.logit_scale if S.logit_scale != 1.0 else logits
+
+    def _layer_runs(self):
+        """(run index, layer spec, weights, weights of the next run or None)
+        in the order the layers run; looped layers come once per pass, and
+        caches and states are keyed by the run."""
+        S, M = self.spec, self.model
+        runs = S.runs
+        for r, i in enumerate(runs):
+            yield (r, S.layers[i], M.layers[i],
+                   M.layers[runs[r + 1]] if r + 1 < len(runs) else None)
 
     def _layers_parallel_gated(self, tokens, meta, capture):
         """One norm per layer feeds the mixer (through the block's short
@@ -550,9 +579,8 @@ class HybridEngine:
         eps, mult = S.norm_eps, S.residual_mult
         shared = {}
         x, _ = SM.offset_rmsnorm(M.embed[tokens], M.embed_norm_w, eps, dt)
-        h32, hb = SM.offset_rmsnorm(x, M.layers[0].norm_w, eps, dt)
-        last = S.num_layers - 1
-        for i, (ls, L) in enumerate(zip(S.layers, M.layers)):
+        h32, hb = SM.offset_rmsnorm(x, M.layers[S.runs[0]].norm_w, eps, dt)
+        for i, ls, L, nxt in self._layer_runs():
             if S.conv_taps:
                 hm = SM.causal_tap_conv(h32, L.conv_w, self.slots.tails[i],
                                         meta["cu"], meta["tok_seq"],
@@ -566,10 +594,9 @@ class HybridEngine:
                 f, f2 = self._ff(ls.mlp, L, hb)
                 if f2 is not None:
                     f = f.float() + f2.float()
-            if i < last:
+            if nxt is not None:
                 h32, hb = SM.gated_residual_norm(
-                    x, y, f, gates, L.gate_b, mult, M.layers[i + 1].norm_w,
-                    eps, dt)
+                    x, y, f, gates, L.gate_b, mult, nxt.norm_w, eps, dt)
             else:
                 SM.gated_residual_add(x, y, f, gates, L.gate_b, mult)
             if capture is not None:
@@ -585,11 +612,10 @@ class HybridEngine:
         eps = S.norm_eps
         shared = {}
         x = M.embed[tokens].float()
-        _, hb = SM.offset_rmsnorm(x, M.layers[0].norm_w, eps, dt)
-        last = S.num_layers - 1
-        for i, (ls, L) in enumerate(zip(S.layers, M.layers)):
+        _, hb = SM.offset_rmsnorm(x, M.layers[S.runs[0]].norm_w, eps, dt)
+        for i, ls, L, after in self._layer_runs():
             y = self._mixer(i, ls, L, hb, meta, shared)[0]
-            nxt = M.layers[i + 1].norm_w if i < last else None
+            nxt = after.norm_w if after is not None else None
             hb = SM.sandwich_residual_norm(
                 x, y, None, L.post_w,
                 L.ff_norm_w if ls.mlp is not None else nxt, eps, dt)
@@ -614,7 +640,7 @@ class HybridEngine:
         if S.embed_scale != 1.0:
             x = x * S.embed_scale
         hb = x.to(dt)
-        for i, (ls, L) in enumerate(zip(S.layers, M.layers)):
+        for i, ls, L, _ in self._layer_runs():
             y, y2, (a, b) = self._mixer(i, ls, L, hb, meta, shared, x32=x)
             hb = SM.sandwich_residual_norm(x, y, y2, L.post_w, None, eps, dt,
                                            off, a, b, cast_next=True)
@@ -637,11 +663,10 @@ class HybridEngine:
         x = M.embed[tokens].float()
         if S.embed_scale != 1.0:
             x = x * S.embed_scale
-        _, hb = SM.offset_rmsnorm(x, M.layers[0].norm_w, eps, dt, off, ng)
-        last = S.num_layers - 1
-        for i, (ls, L) in enumerate(zip(S.layers, M.layers)):
+        _, hb = SM.offset_rmsnorm(x, M.layers[S.runs[0]].norm_w, eps, dt, off, ng)
+        for i, ls, L, after in self._layer_runs():
             y = self._mixer(i, ls, L, hb, meta, shared)[0]
-            nxt = M.layers[i + 1].norm_w if i < last else None
+            nxt = after.norm_w if after is not None else None
             hb = SM.residual_add_norm(
                 x, y, L.ff_norm_w if ls.mlp is not None else nxt, eps, dt, off, ng)
             if ls.mlp is not None:
@@ -649,6 +674,39 @@ class HybridEngine:
                 hb = SM.residual_add_norm(x, f, nxt, eps, dt, off, ng)
             if capture is not None:
                 capture.append(x.clone())
+        return x
+
+    def _layers_hyper(self, tokens, meta, capture):
+        """Residual streams x_1 .. x_S: a sublayer reads the norm of a
+        weighted sum of them, then every stream becomes a mix of the old ones
+        plus its share of the output. One kernel per sublayer closes it (the
+        norms of a pair's two sides, stream update) and opens the next (read
+        sum and norm)."""
+        S, M, dt = self.spec, self.model, self.dtype
+        eps, ctr = S.norm_eps, S.norm_center
+        shared = {}
+        first = M.layers[S.runs[0]]
+        x, hb = SM.hyper_start(M.embed, tokens, S.embed_scale, S.streams,
+                               first.hc1_in, first.norm_w, eps, dt, ctr)
+        for i, ls, L, after in self._layer_runs():
+            y, y2, (a, b) = self._mixer(i, ls, L, hb, meta, shared)
+            normed = y2 is not None and ls.mixer.out_norm
+            nxt = ((L.hc2_in, L.ff_norm_w) if ls.mlp is not None
+                   else (after.hc1_in, after.norm_w) if after is not None
+                   else (None, None))
+            hb = SM.hyper_residual_norm(
+                x, y, y2, L.left_norm_w if normed else None,
+                L.right_norm_w if normed else None, a, b, L.hc1_mix, L.hc1_out,
+                *nxt, eps, dt, ctr)
+            if ls.mlp is not None:
+                f, f2 = self._ff(ls.mlp, L, hb)
+                nxt = ((after.hc1_in, after.norm_w) if after is not None
+                       else (None, None))
+                hb = SM.hyper_residual_norm(x, f, f2, None, None, 1.0, 1.0,
+                                            L.hc2_mix, L.hc2_out, *nxt, eps, dt,
+                                            ctr)
+            if capture is not None:
+                capture.append(x.sum(1))
         return x
 
     def score(self, ids: Seq[int]) -> torch.Tensor:

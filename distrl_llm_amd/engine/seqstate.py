@@ -6,14 +6,16 @@ come and go:
 * :class:`LatentCachePool` — paged rows for every attention layer that owns
   a cache: ``[latent | rotated key part]`` for latent attention (layers
   that read another layer's cache own none), ``[keys of all kv heads |
-  values of all kv heads]`` for grouped-query attention. Block ids come
+  values of all kv heads]`` for grouped-query attention (differential
+  attention holds two key maps per kv head). Block ids come
   from the same refcounting :class:`BlockAllocator` as the dense models'
   K/V pool, so a forked candidate shares its prompt's full pages.
-  Tensors are keyed by mixer unit: the layer index, or (layer, side) for
-  the two sides of a parallel pair.
+  Tensors are keyed by mixer unit: the index of the layer run (the layer
+  index unless layers are looped), or (run, side) for the two sides of a
+  parallel pair.
 * :class:`StateSlotPool` — fixed-size fp32 state per live sequence: the
   last ``taps - 1`` inputs of every short convolution (the block's own, or
-  a delta-rule layer's over its q/k/v channels) and the state of every
+  a delta-rule or attention layer's over its q/k/v channels) and the state of every
   recurrent layer (a vector for minGRU, a matrix per head for the delta
   rule). A slot is zeroed when it is handed out, so whatever its previous
   owner left cannot leak.
@@ -28,7 +30,7 @@ import torch
 from ..models.hybrid import (DeltaRuleSpec, HybridSpec, LatentAttentionSpec,
                              MinGRUSpec, SigmoidAttentionSpec,
                              SinkAttentionSpec, WindowAttentionSpec,
-                             mixer_units)
+                             mixer_conv, mixer_units)
 from .kvcache import BlockAllocator
 
 
@@ -55,7 +57,7 @@ class LatentCachePool:
                 or (isinstance(m, LatentAttentionSpec) and m.kv_from is None))
 
     def layer_rows(self, spec: HybridSpec, layer: int) -> torch.Tensor:
-        return self.unit_rows(layer, spec.layers[layer].mixer)
+        return self.unit_rows(layer, spec.layers[spec.runs[layer]].mixer)
 
     def unit_rows(self, key, m) -> torch.Tensor:
         src = getattr(m, "kv_from", None)
@@ -82,10 +84,10 @@ class StateSlotPool:
         self.num_slots = num_slots
         self.scratch_slot = num_slots     # never handed out (padding rows)
         D, k = spec.width, max(spec.conv_taps - 1, 0)
-        # conv tails: one tensor per layer, [slots + 1, taps-1, width] fp32
+        # conv tails: one tensor per layer run, [slots + 1, taps-1, width] fp32
         self.tails: List[torch.Tensor] = [
             torch.zeros(num_slots + 1, k, D, dtype=torch.float32, device=device)
-            for _ in spec.layers]
+            for _ in spec.runs]
         # recurrent state: mixer unit -> [slots + 1, state size] fp32
         self.recurrent: Dict[object, torch.Tensor] = {
             i: torch.zeros(num_slots + 1, m.state_size, dtype=torch.float32,
@@ -95,10 +97,9 @@ class StateSlotPool:
         # a mixer's own short convolution: mixer unit ->
         # [slots + 1, taps - 1, channels] fp32
         self.mixer_tails: Dict[object, torch.Tensor] = {
-            i: torch.zeros(num_slots + 1, m.taps - 1, m.conv_channels,
+            i: torch.zeros(num_slots + 1, mixer_conv(m)[0] - 1, mixer_conv(m)[1],
                            dtype=torch.float32, device=device)
-            for i, m in mixer_units(spec)
-            if isinstance(m, DeltaRuleSpec)}
+            for i, m in mixer_units(spec) if mixer_conv(m) is not None}
         self._free = list(range(num_slots - 1, -1, -1))
 
     @property

@@ -71,6 +71,23 @@ parameter, so another design can reuse them in another order.
 * feed-forward: a plain two-matrix MLP with tanh-GELU, or a mixture of
   SiLU-gated experts routed by sigmoid scores that are not renormalised and
   scale the expert's *input*.
+
+``Sagedra`` is the fifth:
+
+* several residual streams in fp32 (hyper-connections): a sublayer reads the
+  layer norm (mean taken off, plain weight) of a learned weighted sum of the
+  streams, and every stream becomes a learned mix of the old ones plus its
+  share of the sublayer's output; a stretch of layers runs several times in
+  a row with the same weights and a cache or state per pass; scaled
+  embedding, separate output matrix, tanh-capped logits;
+* mixers: differential attention (two softmax maps per head over the same
+  values, the second taken off the first with a learned factor, the
+  difference RMS-normed per head; biases, a short causal convolution on q, k
+  and v, queries scaled with the position) and a parallel pair whose sides
+  are RMS-normed before they are summed: sliding-window attention (half
+  rotary with rescaled frequencies, q/k RMS-normed after it, a sigmoid gate
+  per output entry) beside the per-head gated delta rule;
+* feed-forward: a dense tanh-GELU GLU.
 """
 
 from __future__ import annotations
@@ -83,6 +100,8 @@ from typing import Dict, List, Optional
 
 import torch
 import torch.nn as nn
+
+from ..ops.seqmix import MAX_STREAMS
 
 
 # ------------------------------------------------------------------ specs
@@ -271,7 +290,17 @@ class WindowAttentionSpec:
     i + dims/2) on the first ``rope_dims`` entries with optionally rescaled
     frequencies, mixing of the heads' scores by a learned [H, H] matrix
     before the softmax, a distance bias ``-r1_h ln(1 + r2_h (i - j))`` and a
-    per-head sigmoid gate read from the mixer input."""
+    sigmoid gate read from the mixer input, one per head or
+    (``entry_gate``) one per output entry.
+
+    Further options: a short causal convolution on the projected q/k/v
+    channels (``conv_taps``), a weightless RMS norm of q and k after the
+    rotation (``qk_unit``), queries scaled by
+    ``1 + coef ln(floor((p + 1) / every) + 1)`` (``q_temp``), a bias on the
+    output projection, and ``maps`` = 2: differential attention, where every
+    head has two query/key maps over the same values and gives
+    ``N(a1 - lambda a2) (1 - diff)``, N a weightless RMS norm over the head's
+    values and ``lambda = e^(lq1.lk1) - e^(lq2.lk2) + diff``."""
     heads: int
     kv_heads: int
     dim: int
@@ -287,25 +316,41 @@ class WindowAttentionSpec:
     score_mix: bool = False
     log_distance: bool = False
     out_gate: bool = False
+    entry_gate: bool = False
+    conv_taps: int = 0                  # 0 = no convolution
+    qk_unit: bool = False
+    q_temp: Optional[tuple] = None      # (coef, every)
+    out_bias: bool = False
+    maps: int = 1
+    diff: float = 0.0
 
     kind = "window_attention"
 
     @property
-    def q_size(self) -> int:
-        return self.heads * self.dim
+    def q_size(self) -> int:           # head by head, map by map
+        return self.heads * self.maps * self.dim
 
     @property
     def k_size(self) -> int:
-        return self.kv_heads * self.dim
+        return self.kv_heads * self.maps * self.dim
 
     @property
     def v_size(self) -> int:
         return self.kv_heads * self.vdim
 
     @property
+    def conv_channels(self) -> int:    # q | k | v, convolved together
+        return self.q_size + self.k_size + self.v_size
+
+    @property
+    def gate_size(self) -> int:
+        if self.entry_gate:
+            return self.heads * self.vdim
+        return self.heads if self.out_gate else 0
+
+    @property
     def in_size(self) -> int:          # [q | k | v | gate]
-        return (self.q_size + self.k_size + self.v_size
-                + (self.heads if self.out_gate else 0))
+        return self.conv_channels + self.gate_size
 
     @property
     def cache_width(self) -> int:      # one cache row = [k heads | v heads]
@@ -319,11 +364,13 @@ class WindowAttentionSpec:
 @dataclass(frozen=True)
 class ParallelMixerSpec:
     """Two mixers that read the same input; the result is
-    ``left_scale * left + right_scale * right``."""
+    ``left_scale * left + right_scale * right``, with ``out_norm`` each side
+    RMS-normed over the width first (plain weights)."""
     left: object
     right: object
     left_scale: float
     right_scale: float
+    out_norm: bool = False
 
     kind = "parallel"
 
@@ -333,15 +380,26 @@ class ParallelMixerSpec:
 
 
 def mixer_units(spec: "HybridSpec"):
-    """Every mixer that owns cache rows or state, with its key: the layer
-    index, or (layer index, side) for the sides of a parallel pair."""
-    for i, ls in enumerate(spec.layers):
-        m = ls.mixer
+    """Every mixer that owns cache rows or state, with its key: the index of
+    the layer run (the layer index, unless layers are looped: every pass is a
+    unit of its own), or (run index, side) for the sides of a parallel
+    pair."""
+    for i, layer in enumerate(spec.runs):
+        m = spec.layers[layer].mixer
         if isinstance(m, ParallelMixerSpec):
             yield (i, 0), m.left
             yield (i, 1), m.right
         else:
             yield i, m
+
+
+def mixer_conv(m):
+    """(taps, channels) of a mixer's own short convolution, or None."""
+    if isinstance(m, DeltaRuleSpec):
+        return m.taps, m.conv_channels
+    if isinstance(m, WindowAttentionSpec) and m.conv_taps:
+        return m.conv_taps, m.conv_channels
+    return None
 
 
 def rotary_frequencies(dims: int, base: float, scaling: Optional[tuple] = None):
@@ -350,10 +408,26 @@ def rotary_frequencies(dims: int, base: float, scaling: Optional[tuple] = None):
     that turn fewer than ``slow`` times over ``original`` positions are
     slowed by ``factor``, those that turn more than ``fast`` times are kept,
     the ones between are blended linearly over the pair index, and cos/sin
-    grow by ``0.1 ln(factor) + 1``."""
+    grow by ``0.1 ln(factor) + 1``. With
+    ``scaling = ("wavelength", factor, low, high, original)`` pairs whose
+    wavelength is below ``original / high`` are kept, those above
+    ``original / low`` are slowed by ``factor``, the ones between are blended
+    linearly over ``original / wavelength``; cos/sin keep their size."""
     half = dims // 2
     f = [float(base) ** (-2.0 * i / dims) for i in range(half)]
     if not scaling:
+        return f, 1.0
+    if scaling[0] == "wavelength":
+        factor, low, high, original = (float(v) for v in scaling[1:])
+        for i in range(half):
+            turns = original * f[i] / (2.0 * math.pi)      # original / wavelength
+            if turns > high:
+                continue
+            if turns < low:
+                f[i] /= factor
+            else:
+                keep = (turns - low) / (high - low) if high > low else 1.0
+                f[i] = (1.0 - keep) * f[i] / factor + keep * f[i]
         return f, 1.0
     factor, original, fast, slow = (float(v) for v in scaling)
 
@@ -372,7 +446,8 @@ def rotary_frequencies(dims: int, base: float, scaling: Optional[tuple] = None):
 class GluSpec:
     """Gated linear unit. ``act`` "capped": g = min(gate, limit),
     u = clamp(up, +-limit), y = g * sigmoid(1.702 g) * (u + 1); "silu":
-    y = silu(gate) * up (limit unused)."""
+    y = silu(gate) * up; "gelu_tanh": y = gelu_tanh(gate) * up (limit unused
+    by both)."""
     ff: int
     limit: float = 0.0
     act: str = "capped"
@@ -422,7 +497,9 @@ class HybridSpec:
     # "parallel_gated": one norm feeds mixer and feed-forward, gated sum;
     # "sandwich": norm before and after each sublayer, one after the other;
     # "post_norm": sublayers read the residual, only their output is normed;
-    # "pre_norm": x += sublayer(norm(x)), nothing else
+    # "pre_norm": x += sublayer(norm(x)), nothing else;
+    # "hyper": ``streams`` residual streams, u = sum_s in[s] x_s,
+    # x_t <- sum_s mix[s, t] x_s + out[t] sublayer(norm(u))
     block: str = "parallel_gated"
     design: str = "nibalix"
     norm_offset: float = 1.0    # norm weights act as (offset + w)
@@ -432,10 +509,25 @@ class HybridSpec:
     # norms are taken separately over this many equal consecutive parts of
     # the width
     norm_groups: int = 1
+    norm_center: bool = False   # layer norm: the mean is taken off first
+    streams: int = 1            # residual streams of the "hyper" block
+    logit_softcap: float = 0.0  # > 0: logits <- cap tanh(logits / cap)
+    # (start, stop, times): layers start .. stop - 1 run ``times`` times in a
+    # row, every pass with a cache or state of its own
+    loop: Optional[tuple] = None
 
     @property
     def num_layers(self) -> int:
         return len(self.layers)
+
+    @property
+    def runs(self) -> tuple:
+        """Layer indices in the order they run."""
+        n = len(self.layers)
+        if self.loop is None:
+            return tuple(range(n))
+        a, b, times = self.loop
+        return (tuple(range(a)) + tuple(range(a, b)) * times + tuple(range(b, n)))
 
 
 def nibalix_spec_from_config(cfg: dict, name: str = "nibalix") -> HybridSpec:
@@ -562,6 +654,12 @@ def _make_mixer_weights(mod, m, D, P, packed_input=True):
             mod.talk = P(m.heads, m.heads, dt=f32)
         if m.log_distance:
             mod.dist_r1, mod.dist_r2 = P(m.heads, dt=f32), P(m.heads, dt=f32)
+        if m.conv_taps:
+            mod.conv_w = P(m.conv_channels, m.conv_taps, dt=f32)
+        if m.maps == 2:
+            mod.lam_w = P(4, m.dim, dt=f32)     # lq1, lk1, lq2, lk2
+        if m.out_bias:
+            mod.out_b = P(D)
         mod.out_w = P(D, m.heads * m.vdim)
     elif isinstance(m, DeltaRuleSpec):
         mod.conv_w = P(m.conv_channels, m.taps, dt=f32)
@@ -608,6 +706,16 @@ class HybridLayer(nn.Module):
             self.norm_w = P(D, dt=f32)
             if ls.mlp is not None:
                 self.ff_norm_w = P(D, dt=f32)
+        elif spec.block == "hyper":
+            # per sublayer q: stream weights in/out [S] and mix [from, to]
+            n = spec.streams
+            self.norm_w = P(D, dt=f32)
+            self.hc1_in, self.hc1_out = P(n, dt=f32), P(n, dt=f32)
+            self.hc1_mix = P(n, n, dt=f32)
+            if ls.mlp is not None:
+                self.ff_norm_w = P(D, dt=f32)
+                self.hc2_in, self.hc2_out = P(n, dt=f32), P(n, dt=f32)
+                self.hc2_mix = P(n, n, dt=f32)
         elif spec.block == "sandwich":
             self.norm_w = P(D, dt=f32)
             self.post_w = P(D, dt=f32)
@@ -626,6 +734,8 @@ class HybridLayer(nn.Module):
             self.left, self.right = nn.Module(), nn.Module()
             _make_mixer_weights(self.left, m.left, D, P, packed_input=False)
             _make_mixer_weights(self.right, m.right, D, P, packed_input=False)
+            if m.out_norm:
+                self.left_norm_w, self.right_norm_w = P(D, dt=f32), P(D, dt=f32)
         else:
             _make_mixer_weights(self, m, D, P)
         f = ls.mlp
@@ -682,12 +792,11 @@ class HybridLM(nn.Module):
         """{checkpoint tensor name: (packed parameter, row0, rows | None)}.
         ``rows`` None means the tensor fills the whole parameter; expert
         entries carry an index tuple instead of a row range."""
-        if self.spec.design == "nedasun":
-            return _nedasun_named_slices(self)
-        if self.spec.design == "kakilorn":
-            return _kakilorn_named_slices(self)
-        if self.spec.design == "legilix":
-            return _legilix_named_slices(self)
+        table = {"nedasun": _nedasun_named_slices, "kakilorn": _kakilorn_named_slices,
+                 "legilix": _legilix_named_slices,
+                 "sagedra": _sagedra_named_slices}.get(self.spec.design)
+        if table is not None:
+            return table(self)
         out = {"embed": (self.embed, None), "embed.norm": (self.embed_norm_w, None),
                "final.norm": (self.final_norm_w, None), "head": (self.head, None)}
         D = self.spec.width
@@ -777,6 +886,12 @@ class HybridLM(nn.Module):
                 r = 0.3 + 0.1 * r
             elif last in ("r1", "r2"):
                 r = 0.5 + 0.1 * r.abs()
+            elif ".hc" in name:         # streams: read evenly, kept nearly apart
+                n = self.spec.streams
+                r = (torch.eye(n, device=dev) + 0.05 * r if last == "mix"
+                     else 0.1 * r + (1.0 / n if last == "in" else 1.0))
+            elif last == "out":         # closing norm of a pair's side
+                r = 1.0 + 0.1 * r
             elif last == "conv":
                 r *= 0.5
             elif dst.dim() >= 2 and "canon" not in name:
@@ -793,29 +908,46 @@ class HybridLM(nn.Module):
 
 # ------------------------------------------------------------ checkpoints
 
-def load_nibalix_checkpoint(path: str, dtype=torch.bfloat16, device=None) -> HybridLM:
+def _load_design(path: str, design: str, to_spec, dtype, device,
+                 optional=None) -> HybridLM:
+    """Build a design's model from ``config.json`` (``to_spec(cfg, name)``)
+    and fill it from ``model.safetensors``. Tensors the design does not name
+    are reported and left out; ``optional(spec)`` names tensors that a
+    checkpoint may leave out."""
     from safetensors.torch import load_file
     with open(os.path.join(path, "config.json")) as f:
         cfg = json.load(f)
-    name = os.path.basename(os.path.normpath(path)) or "nibalix"
-    model = HybridLM(nibalix_spec_from_config(cfg, name), dtype=dtype, device=device)
+    name = os.path.basename(os.path.normpath(path)) or design
+    model = HybridLM(to_spec(cfg, name), dtype=dtype, device=device)
     tensors = load_file(os.path.join(path, "model.safetensors"))
     known = model._named_slices()
     extra = sorted(k for k in tensors if k not in known)
     if extra:
         import sys
-        sys.stderr.write(f"[nibalix] ignoring {len(extra)} tensors the design "
+        sys.stderr.write(f"[{design}] ignoring {len(extra)} tensors the design "
                          f"does not name: {extra[:4]}\n")
-    model.load_tensors({k: v for k, v in tensors.items() if k in known})
+    have = {k: v for k, v in tensors.items() if k in known}
+    missing = set(known) - set(have) - (optional(model.spec) if optional else set())
+    if missing:
+        raise ValueError(f"checkpoint misses tensors: {sorted(missing)[:8]}")
+    model.load_tensors(have, strict=False)
     return model
 
 
-def save_nibalix_checkpoint(model: HybridLM, path: str) -> None:
+def _save_design(model: HybridLM, path: str, to_config) -> None:
     from safetensors.torch import save_file
     os.makedirs(path, exist_ok=True)
     save_file(model.export_tensors(), os.path.join(path, "model.safetensors"))
     with open(os.path.join(path, "config.json"), "w") as f:
-        json.dump(nibalix_config_from_spec(model.spec), f, indent=1)
+        json.dump(to_config(model.spec), f, indent=1)
+
+
+def load_nibalix_checkpoint(path: str, dtype=torch.bfloat16, device=None) -> HybridLM:
+    return _load_design(path, "nibalix", nibalix_spec_from_config, dtype, device)
+
+
+def save_nibalix_checkpoint(model: HybridLM, path: str) -> None:
+    _save_design(model, path, nibalix_config_from_spec)
 
 
 # ---------------------------------------------------------------- Nedasun
@@ -963,36 +1095,18 @@ def _nedasun_named_slices(model: "HybridLM") -> Dict[str, tuple]:
 
 
 def load_nedasun_checkpoint(path: str, dtype=torch.bfloat16, device=None) -> HybridLM:
-    from safetensors.torch import load_file
-    with open(os.path.join(path, "config.json")) as f:
-        cfg = json.load(f)
-    name = os.path.basename(os.path.normpath(path)) or "nedasun"
-    model = HybridLM(nedasun_spec_from_config(cfg, name), dtype=dtype, device=device)
-    tensors = load_file(os.path.join(path, "model.safetensors"))
-    known = model._named_slices()
-    extra = sorted(k for k in tensors if k not in known)
-    if extra:
-        import sys
-        sys.stderr.write(f"[nedasun] ignoring {len(extra)} tensors the design "
-                         f"does not name: {extra[:4]}\n")
     # the blend factor is read only by mixing layers after the first one: a
     # checkpoint may leave it out elsewhere
-    unused = {f"l{i}.mix.vmix" for i, ls in enumerate(model.spec.layers)
-              if isinstance(ls.mixer, SinkAttentionSpec) and ls.mixer.v_first is None}
-    have = {k: v for k, v in tensors.items() if k in known}
-    missing = set(known) - set(have) - unused
-    if missing:
-        raise ValueError(f"checkpoint misses tensors: {sorted(missing)[:8]}")
-    model.load_tensors(have, strict=False)
-    return model
+    def optional(spec):
+        return {f"l{i}.mix.vmix" for i, ls in enumerate(spec.layers)
+                if isinstance(ls.mixer, SinkAttentionSpec) and ls.mixer.v_first is None}
+
+    return _load_design(path, "nedasun", nedasun_spec_from_config, dtype, device,
+                        optional)
 
 
 def save_nedasun_checkpoint(model: HybridLM, path: str) -> None:
-    from safetensors.torch import save_file
-    os.makedirs(path, exist_ok=True)
-    save_file(model.export_tensors(), os.path.join(path, "model.safetensors"))
-    with open(os.path.join(path, "config.json"), "w") as f:
-        json.dump(nedasun_config_from_spec(model.spec), f, indent=1)
+    _save_design(model, path, nedasun_config_from_spec)
 
 
 # --------------------------------------------------------------- Kakilorn
@@ -1184,30 +1298,13 @@ def _safetensors_shapes(path: str) -> dict:
 
 
 def load_kakilorn_checkpoint(path: str, dtype=torch.bfloat16, device=None) -> HybridLM:
-    from safetensors.torch import load_file
-    with open(os.path.join(path, "config.json")) as f:
-        cfg = json.load(f)
-    name = os.path.basename(os.path.normpath(path)) or "kakilorn"
-    file = os.path.join(path, "model.safetensors")
-    spec = kakilorn_spec_from_config(cfg, name, _safetensors_shapes(file))
-    model = HybridLM(spec, dtype=dtype, device=device)
-    tensors = load_file(file)
-    known = model._named_slices()
-    extra = sorted(k for k in tensors if k not in known)
-    if extra:
-        import sys
-        sys.stderr.write(f"[kakilorn] ignoring {len(extra)} tensors the design "
-                         f"does not name: {extra[:4]}\n")
-    model.load_tensors({k: v for k, v in tensors.items() if k in known})
-    return model
+    shapes = _safetensors_shapes(os.path.join(path, "model.safetensors"))
+    return _load_design(path, "kakilorn", lambda cfg, name: kakilorn_spec_from_config(
+        cfg, name, shapes), dtype, device)
 
 
 def save_kakilorn_checkpoint(model: HybridLM, path: str) -> None:
-    from safetensors.torch import save_file
-    os.makedirs(path, exist_ok=True)
-    save_file(model.export_tensors(), os.path.join(path, "model.safetensors"))
-    with open(os.path.join(path, "config.json"), "w") as f:
-        json.dump(kakilorn_config_from_spec(model.spec), f, indent=1)
+    _save_design(model, path, kakilorn_config_from_spec)
 
 
 # ---------------------------------------------------------------- Legilix
@@ -1337,25 +1434,172 @@ def _legilix_named_slices(model: "HybridLM") -> Dict[str, tuple]:
 
 
 def load_legilix_checkpoint(path: str, dtype=torch.bfloat16, device=None) -> HybridLM:
-    from safetensors.torch import load_file
-    with open(os.path.join(path, "config.json")) as f:
-        cfg = json.load(f)
-    name = os.path.basename(os.path.normpath(path)) or "legilix"
-    model = HybridLM(legilix_spec_from_config(cfg, name), dtype=dtype, device=device)
-    tensors = load_file(os.path.join(path, "model.safetensors"))
-    known = model._named_slices()
-    extra = sorted(k for k in tensors if k not in known)
-    if extra:
-        import sys
-        sys.stderr.write(f"[legilix] ignoring {len(extra)} tensors the design "
-                         f"does not name: {extra[:4]}\n")
-    model.load_tensors({k: v for k, v in tensors.items() if k in known})
-    return model
+    return _load_design(path, "legilix", legilix_spec_from_config, dtype, device)
 
 
 def save_legilix_checkpoint(model: HybridLM, path: str) -> None:
-    from safetensors.torch import save_file
-    os.makedirs(path, exist_ok=True)
-    save_file(model.export_tensors(), os.path.join(path, "model.safetensors"))
-    with open(os.path.join(path, "config.json"), "w") as f:
-        json.dump(legilix_config_from_spec(model.spec), f, indent=1)
+    _save_design(model, path, legilix_config_from_spec)
+
+
+# ---------------------------------------------------------------- Sagedra
+
+def _heads_from_config(i, mc):
+    heads, kvh = int(mc["heads"]), int(mc["kv_heads"])
+    if kvh < 1 or heads < 1 or heads % kvh:
+        raise ValueError(f"layer {i}: heads must be a multiple of kv_heads")
+    return dict(heads=heads, kv_heads=kvh, dim=int(mc["dim"]), vdim=int(mc["vdim"]))
+
+
+def sagedra_spec_from_config(cfg: dict, name: str = "sagedra") -> HybridSpec:
+    """Map a Sagedra ``config.json`` onto the generic layer specs."""
+    layers = []
+    for i, lc in enumerate(cfg["layers"]):
+        mc, typ = lc["mixer"], lc["type"]
+        if typ == "attention":
+            qt = mc.get("q_temp")
+            mixer = WindowAttentionSpec(
+                **_heads_from_config(i, mc), scale=float(mc["scale"]),
+                qkv_bias=True, out_bias=True, conv_taps=int(mc["conv"]), maps=2,
+                diff=float(mc["diff"]),
+                q_temp=(float(qt["coef"]), float(qt["every"])) if qt else None)
+            if mixer.conv_taps < 1:
+                raise ValueError(f"layer {i}: conv needs at least one tap")
+            if mixer.q_temp is not None and mixer.q_temp[1] <= 0:
+                raise ValueError(f"layer {i}: q_temp.every must be positive")
+        elif typ == "parallel":
+            lm, rm = mc["left"], mc["right"]
+            rot = lm.get("rot") or {}
+            sc = rot.get("scaling")
+            left = WindowAttentionSpec(
+                **_heads_from_config(i, lm), scale=float(lm["scale"]),
+                window=int((lm.get("mask") or {}).get("size") or 0),
+                rope_dims=int(rot.get("dims") or 0),
+                rope_base=float(rot.get("base") or 10000.0),
+                rope_scaling=(None if not sc else
+                              ("wavelength", float(sc["factor"]), float(sc["low"]),
+                               float(sc["high"]), float(sc["original"]))),
+                qk_unit=True, entry_gate=True)
+            if left.rope_dims > left.dim or left.rope_dims % 2:
+                raise ValueError(f"layer {i}: rot.dims must be even and <= dim")
+            mixer = ParallelMixerSpec(left, _delta_from_config(i, rm, False),
+                                      0.5, 0.5, out_norm=True)
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {typ!r}")
+        fc, mlp = lc.get("mlp"), None
+        if fc is not None:
+            if fc.get("kind") != "dense":
+                raise ValueError(f"layer {i}: unknown mlp kind {fc.get('kind')!r}")
+            mlp = GluSpec(ff=int(fc["ff"]), act="gelu_tanh")
+        layers.append(LayerSpec(mixer, mlp))
+    loop = cfg.get("loop")
+    if loop:
+        loop = (int(loop["start"]), int(loop["stop"]), int(loop["times"]))
+        if not (0 <= loop[0] <= loop[1] <= len(layers)) or loop[2] < 1:
+            raise ValueError("loop: needs 0 <= start <= stop <= layers and times >= 1")
+    streams = int(cfg.get("streams") or 1)
+    if not 1 <= streams <= MAX_STREAMS:
+        raise ValueError(f"streams must be in [1, {MAX_STREAMS}]")
+    return HybridSpec(name=name, vocab_size=int(cfg["vocab"]),
+                      width=int(cfg["width"]),
+                      norm_eps=float(cfg["norm"]["eps"]), residual_mult=1.0,
+                      conv_taps=0, layers=tuple(layers), block="hyper",
+                      design="sagedra", norm_offset=0.0, norm_center=True,
+                      embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)),
+                      streams=streams, loop=loop or None,
+                      logit_softcap=float(cfg.get("logit_softcap") or 0.0))
+
+
+def sagedra_config_from_spec(spec: HybridSpec) -> dict:
+    """Inverse of :func:`sagedra_spec_from_config` (checkpoint saving)."""
+    layers = []
+    for ls in spec.layers:
+        m = ls.mixer
+        if isinstance(m, ParallelMixerSpec):
+            a, d = m.left, m.right
+            rot = {"base": a.rope_base, "dims": a.rope_dims}
+            if a.rope_scaling:
+                rot["scaling"] = dict(zip(("factor", "low", "high", "original"),
+                                          a.rope_scaling[1:]))
+            left = {"heads": a.heads, "kv_heads": a.kv_heads, "dim": a.dim,
+                    "vdim": a.vdim, "scale": a.scale, "rot": rot}
+            if a.window:
+                left["mask"] = {"size": a.window}
+            mc = {"left": left,
+                  "right": {"heads": d.heads, "kv_heads": d.kv_heads, "dim": d.dim,
+                            "vdim": d.vdim, "conv": d.taps}}
+            typ = "parallel"
+        else:
+            mc = {"heads": m.heads, "kv_heads": m.kv_heads, "dim": m.dim,
+                  "vdim": m.vdim, "scale": m.scale, "conv": m.conv_taps,
+                  "diff": m.diff}
+            if m.q_temp:
+                mc["q_temp"] = {"coef": m.q_temp[0], "every": m.q_temp[1]}
+            typ = "attention"
+        fc = None if ls.mlp is None else {"kind": "dense", "ff": ls.mlp.ff}
+        layers.append({"type": typ, "mixer": mc, "mlp": fc})
+    out = {"architecture": "Sagedra", "embedding": {"scale": spec.embed_scale},
+           "layers": layers, "norm": {"eps": spec.norm_eps}, "streams": spec.streams,
+           "vocab": spec.vocab_size, "width": spec.width}
+    if spec.logit_softcap:
+        out["logit_softcap"] = spec.logit_softcap
+    if spec.loop:
+        out["loop"] = dict(zip(("start", "stop", "times"), spec.loop))
+    return out
+
+
+def _sagedra_named_slices(model: "HybridLM") -> Dict[str, tuple]:
+    out = {"embed": (model.embed, None), "final.norm": (model.final_norm_w, None),
+           "head": (model.head, None)}
+    for i, (ls, L) in enumerate(zip(model.spec.layers, model.layers)):
+        p, m = f"l{i}.", ls.mixer
+        x = p + "mix."
+        out[p + "norm1"] = (L.norm_w, None)
+        out[p + "hc1.in"], out[p + "hc1.out"] = (L.hc1_in, None), (L.hc1_out, None)
+        out[p + "hc1.mix"] = (L.hc1_mix, None)
+        if isinstance(m, ParallelMixerSpec):
+            a, d, W = m.left, m.right, L.right
+            r0 = 0
+            for nm, rows in (("q", a.q_size), ("k", a.k_size), ("v", a.v_size),
+                             ("g", a.gate_size)):
+                out[x + "left." + nm] = (L.in_w, (r0, rows))
+                r0 += rows
+            out[x + "left.o"] = (L.left.out_w, None)
+            out[x + "left.out"] = (L.left_norm_w, None)
+            out[x + "right.out"] = (L.right_norm_w, None)
+            y, c0 = x + "right.", 0
+            for nm, rows in (("q", d.qk_size), ("k", d.qk_size), ("v", d.v_size)):
+                out[y + nm] = (L.in_w, (r0 + c0, rows))
+                out[y + nm + ".conv"] = (W.conv_w, (c0, rows))
+                c0 += rows
+            out[y + "g"] = (L.in_w, (r0 + c0, d.v_size))
+            out[y + "b"] = (W.ab_w, (0, d.heads))
+            out[y + "a"] = (W.ab_w, (d.heads, d.heads))
+            out[y + "A_log"], out[y + "dt_bias"] = (W.a_log, None), (W.dt_bias, None)
+            out[y + "norm"], out[y + "o"] = (W.onorm_w, None), (W.out_w, None)
+        else:
+            r0 = 0
+            for nm, rows in (("q", m.q_size), ("k", m.k_size), ("v", m.v_size)):
+                out[x + nm] = (L.in_w, (r0, rows))
+                out[x + nm + ".b"] = (L.in_b, (r0, rows))
+                out[x + nm + ".conv"] = (L.conv_w, (r0, rows))
+                r0 += rows
+            for k, nm in enumerate(("lq1", "lk1", "lq2", "lk2")):
+                out[x + nm] = (L.lam_w[k], None)
+            out[x + "o"], out[x + "o.b"] = (L.out_w, None), (L.out_b, None)
+        if ls.mlp is not None:
+            f = ls.mlp
+            out[p + "norm2"] = (L.ff_norm_w, None)
+            out[p + "hc2.in"], out[p + "hc2.out"] = (L.hc2_in, None), (L.hc2_out, None)
+            out[p + "hc2.mix"] = (L.hc2_mix, None)
+            out[p + "mlp.gate"] = (L.gu_w, (0, f.ff))
+            out[p + "mlp.up"] = (L.gu_w, (f.ff, f.ff))
+            out[p + "mlp.down"] = (L.down_w, None)
+    return out
+
+
+def load_sagedra_checkpoint(path: str, dtype=torch.bfloat16, device=None) -> HybridLM:
+    return _load_design(path, "sagedra", sagedra_spec_from_config, dtype, device)
+
+
+def save_sagedra_checkpoint(model: HybridLM, path: str) -> None:
+    _save_design(model, path, sagedra_config_from_spec)

@@ -304,37 +304,49 @@ def moe_experts_glu(h, idx, wts, exp_gu, exp_down, limit):
 # ------------------------------------------- windowed softmax attention, MLP
 
 def qk_prepare_kv_write(proj, heads, kv_heads, dim, vdim, q_norm_w, k_norm_w,
-                        eps, positions, freqs, mag, mix, page_slot, cache):
+                        eps, positions, freqs, mag, mix, page_slot, cache,
+                        maps=1, unit=False, q_temp=None, conv=None):
     """``proj`` rows [q | k | v | ...] may be a column slice of a wider
     matrix. ``q_norm_w``/``k_norm_w`` None: no q/k norm; ``freqs`` None: no
     rotation; ``mix`` (fp32 [H, H]): the returned queries are folded with
-    the score-mixing matrix and span every kv head's key columns."""
+    the score-mixing matrix and span every kv head's key columns. ``maps``:
+    query/key maps per head; ``unit``: weightless RMS norm of q and k after
+    the rotation; ``q_temp`` = (coef, every): queries scaled with their
+    position; ``conv`` = (w fp32 [channels, taps], tails, cu, tok_seq,
+    slots): short causal convolution of the q/k/v channels first, whose tails
+    are advanced (every row of the step holds at least one token)."""
     if proj.is_cuda:
+        w, tails, cu, tok_seq, slots = conv if conv is not None else (None,) * 5
+        coef, every = q_temp if q_temp is not None else (0.0, 1.0)
         return _ext("qk_prepare_kv_write").qk_prepare_kv_write(
             proj, heads, kv_heads, dim, vdim, q_norm_w, k_norm_w, eps,
-            positions, freqs, mag, mix, page_slot, cache)
+            positions, freqs, mag, mix, page_slot, cache, maps, unit, coef,
+            every, w, tails, cu, tok_seq, slots)
     return R.qk_prepare_kv_write(proj, heads, kv_heads, dim, vdim, q_norm_w,
                                  k_norm_w, eps, positions, freqs, mag, mix,
-                                 page_slot, cache)
+                                 page_slot, cache, maps, unit, q_temp, conv)
 
 
 def window_attention(q, cache, heads, kv_heads, dim, vdim, whole_key,
                      block_tables, block_size, cu, tok_seq, positions, scale,
                      window, keep_first, r1, r2, gate, out_dtype, tiles=None,
-                     max_tile=0):
+                     max_tile=0, maps=1, lam_w=None, diff=0.0, eps=0.0):
     """``tiles`` (from :func:`query_tiles` with ``WIDE_QUERY_TILE``) selects
     the tiled MFMA kernel for bf16 prompt portions; steps of few tokens per
     row run one workgroup per (token, kv head, share of the keys), fp32
-    models and odd sizes one wave per (token, head). ``gate`` may be a
-    column slice of a wider matrix."""
+    models and odd sizes one wave per (token, head). ``gate`` ([T, H] or one
+    per entry, [T, H vdim]) may be a column slice of a wider matrix. ``maps``
+    = 2 (with ``lam_w`` fp32 [4, dim], ``diff`` and ``eps``): differential
+    attention, two query/key maps per head over the same values."""
     if q.is_cuda:
         return _ext("window_attention").window_attention(
             q, cache, heads, kv_heads, dim, vdim, whole_key, block_tables,
             block_size, tok_seq, positions, scale, window, keep_first, r1, r2,
-            gate, tiles, max_tile)
+            gate, tiles, max_tile, maps, lam_w, diff, eps)
     return R.window_attention(q, cache, heads, kv_heads, dim, vdim, whole_key,
                               block_tables, block_size, cu, positions, scale,
-                              window, keep_first, r1, r2, gate, out_dtype)
+                              window, keep_first, r1, r2, gate, out_dtype,
+                              maps, lam_w, diff, eps)
 
 
 def gelu_tanh(x):
@@ -355,3 +367,58 @@ def moe_experts_scaled_input(h, idx, wts, exp_gu, exp_down):
         return _ext("moe_experts_scaled_input").moe_experts_scaled_input(
             h, idx, wts, exp_gu, exp_down)
     return R.moe_experts_scaled_input(h, idx, wts, exp_gu, exp_down)
+
+
+def gelu_glu(gu):
+    """Rows [gate | up] -> gelu_tanh(gate) * up."""
+    if gu.is_cuda:
+        return _ext("gelu_glu").gelu_glu(gu)
+    return R.gelu_glu(gu)
+
+
+def cap_logits(z, scale, cap):
+    """fp32 scale * z, then with ``cap`` > 0 cap * tanh(./cap)."""
+    if z.is_cuda:
+        return _ext("cap_logits").cap_logits(z, scale, cap)
+    return R.cap_logits(z, scale, cap)
+
+
+# --------------------------------------------------- hyper-connection streams
+
+MAX_STREAMS = 16
+
+
+def hyper_start(embed, tokens, scale, streams, read_w, norm_w, eps, out_dtype,
+                center):
+    """All streams equal to scale * embed[token]; returns (x fp32 [T, S, D],
+    norm(sum_s read_w[s] x_s) in ``out_dtype``). ``center``: layer norm
+    instead of RMS norm."""
+    if embed.is_cuda:
+        return _ext("hyper_start").hyper_start(
+            embed, tokens, scale, streams, read_w, norm_w, eps,
+            _bf16(out_dtype), center)
+    return R.hyper_start(embed, tokens, scale, streams, read_w, norm_w, eps,
+                         out_dtype, center)
+
+
+def hyper_residual_norm(x, y, y2, y_w, y2_w, y_scale, y2_scale, mix, out_w,
+                        read_w, norm_w, eps, out_dtype, center):
+    """Fused sublayer tail on residual streams (x fp32 [T, S, D], in place):
+    s = y_scale y (+ y2_scale y2), each RMS-normed over the width first where
+    it has a weight; x_t <- sum_s mix[s, t] x_s + out_w[t] s; with ``norm_w``
+    the next sublayer's input norm(sum_s read_w[s] x_s)."""
+    if x.is_cuda:
+        return _ext("hyper_residual_norm").hyper_residual_norm(
+            x, y.contiguous(), None if y2 is None else y2.contiguous(), y_w,
+            y2_w, y_scale, y2_scale, mix, out_w, read_w, norm_w, eps,
+            _bf16(out_dtype), center)
+    return R.hyper_residual_norm(x, y, y2, y_w, y2_w, y_scale, y2_scale, mix,
+                                 out_w, read_w, norm_w, eps, out_dtype, center)
+
+
+def hyper_close_norm(x, rows, norm_w, eps, out_dtype, center):
+    """norm(sum of the streams) of the given rows (int64 indices)."""
+    if x.is_cuda:
+        return _ext("hyper_close_norm").hyper_close_norm(
+            x, rows, norm_w, eps, _bf16(out_dtype), center)
+    return R.hyper_close_norm(x, rows, norm_w, eps, out_dtype, center)

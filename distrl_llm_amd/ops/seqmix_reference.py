@@ -494,27 +494,66 @@ def moe_experts_glu(h, idx, wts, exp_gu, exp_down, limit):
 
 # ------------------------------------------- windowed softmax attention, MLP
 
+def tap_conv(x, w, tails, cu, slots):
+    """fp32 y_t = sum_j w[:, j] * x_(t - taps + 1 + j) per sequence, with
+    the inputs before the portion from ``tails[slot]``, which is advanced."""
+    taps = w.shape[1]
+    x = x.float()
+    out = torch.empty_like(x)
+    cu_l, slots_l = cu.tolist(), slots.tolist()
+    for b, s in enumerate(slots_l):
+        a, e = cu_l[b], cu_l[b + 1]
+        if e == a:
+            continue
+        ext = torch.cat([tails[s], x[a:e]], 0)
+        acc = torch.zeros_like(x[a:e])
+        for j in range(taps):
+            acc += w[:, j] * ext[j:j + e - a]
+        out[a:e] = acc
+        if taps > 1:
+            tails[s] = ext[ext.shape[0] - (taps - 1):]
+    return out
+
+
 def qk_prepare_kv_write(proj, heads, kv_heads, dim, vdim, q_norm_w, k_norm_w,
-                        eps, positions, freqs, mag, mix, page_slot, cache):
-    """From packed [q | k | v | ...] projection rows: optional RMS norm of
+                        eps, positions, freqs, mag, mix, page_slot, cache,
+                        maps=1, unit=False, q_temp=None, conv=None):
+    """From packed [q | k | v | ...] projection rows: optional short causal
+    convolution of the q/k/v channels (``conv`` = (w [channels, taps], tails,
+    cu, tok_seq, slots), tails advanced), optional RMS norm of
     every q and k head (plain shared weights), optional half-layout rotation
     of their first 2 len(freqs) entries by position * freqs with cos and sin
-    scaled by ``mag``, page write of [k | v]. Returns the queries in the
-    projection's dtype: [T, heads, dim], or with ``mix`` (fp32 [H, H])
+    scaled by ``mag``, with ``unit`` a weightless RMS norm of q and k after
+    it, with ``q_temp`` = (coef, every) queries times
+    1 + coef ln(floor((p + 1) / every) + 1), page write of [k | v]. ``maps``:
+    query and key maps per head (differential attention). Returns the queries
+    in the projection's dtype: [T, heads * maps, dim], or with ``mix`` (fp32 [H, H])
     [T, heads, kv_heads * dim], where row h holds, in the columns of kv head
     c, sum over the heads g of c of mix[h, g] q_g: its product with a whole
     key row is the score of head h mixed over all heads."""
     T = proj.shape[0]
-    nq, nk = heads * dim, kv_heads * dim
-    q = proj[:, :nq].float().view(T, heads, dim)
-    k = proj[:, nq:nq + nk].float().view(T, kv_heads, dim)
+    hq, hk = heads * maps, kv_heads * maps
+    nq, nk = hq * dim, hk * dim
+    x = proj[:, :nq + nk + kv_heads * vdim].float()
+    if conv is not None:
+        w, tails, cu, _, slots = conv
+        x = tap_conv(x, w, tails, cu, slots)
+    q = x[:, :nq].reshape(T, hq, dim)
+    k = x[:, nq:nq + nk].reshape(T, hk, dim)
     if q_norm_w is not None:
         q = q * torch.rsqrt(q.pow(2).mean(-1, keepdim=True) + eps) * q_norm_w.float()
         k = k * torch.rsqrt(k.pow(2).mean(-1, keepdim=True) + eps) * k_norm_w.float()
     if freqs is not None and freqs.numel():
         q = _rotate_table(q, positions, freqs, mag, False)
         k = _rotate_table(k, positions, freqs, mag, False)
-    v = proj[:, nq + nk:nq + nk + kv_heads * vdim].float()
+    if unit:
+        q = q * torch.rsqrt(q.pow(2).mean(-1, keepdim=True) + eps)
+        k = k * torch.rsqrt(k.pow(2).mean(-1, keepdim=True) + eps)
+    if q_temp is not None:
+        coef, every = q_temp
+        n = torch.floor((positions.float() + 1.0) / every)
+        q = q * (1.0 + coef * torch.log(n + 1.0))[:, None, None]
+    v = x[:, nq + nk:]
     cache[page_slot.long()] = torch.cat([k.reshape(T, nk), v], -1).to(cache.dtype)
     if mix is not None:
         rep = heads // kv_heads
@@ -526,17 +565,43 @@ def qk_prepare_kv_write(proj, heads, kv_heads, dim, vdim, q_norm_w, k_norm_w,
 
 def window_attention(q, cache, heads, kv_heads, dim, vdim, whole_key,
                      block_tables, block_size, cu, positions, scale, window,
-                     keep_first, r1, r2, gate, out_dtype):
+                     keep_first, r1, r2, gate, out_dtype, maps=1, lam_w=None,
+                     diff=0.0, eps=0.0):
     """Grouped-query softmax attention over paged [k | v] rows.
 
     Query i sees the keys j <= i with i - j < window or j < keep_first
     (window 0: all j <= i). score = q . k * scale, where head h meets the
     keys of its own kv head, or with ``whole_key`` (q rows of kv_heads * dim
     entries) the whole key row; ``r1``/``r2`` (fp32 [H]) take
-    r1 ln(1 + r2 (i - j)) off the score; ``gate`` ([T, H] pre-activations)
-    scales head h's result by its sigmoid. -> [T, H * vdim]."""
+    r1 ln(1 + r2 (i - j)) off the score; ``gate`` ([T, H] or, one per entry,
+    [T, H * vdim] pre-activations) scales the result by its sigmoid.
+
+    ``maps`` = 2, differential attention: q [T, 2 H, dim] and the key columns
+    hold two maps per head over the same values; with lambda =
+    exp(lq1.lk1) - exp(lq2.lk2) + diff (``lam_w`` fp32 [4, dim] = lq1, lk1,
+    lq2, lk2) head h gives o / rms(o) * (1 - diff), o = a1 - lambda a2.
+    -> [T, H * vdim]."""
     T = q.shape[0]
     rep = heads // kv_heads
+    if maps == 2:
+        lq1, lk1, lq2, lk2 = lam_w.float()
+        lam = torch.exp((lq1 * lk1).sum()) - torch.exp((lq2 * lk2).sum()) + diff
+        # map m's keys and its copy of the values as rows of their own
+        nk = 2 * kv_heads * dim
+        v = cache[:, nk:]
+        k = cache[:, :nk].reshape(-1, kv_heads, 2, dim)
+        a = []
+        for m in range(2):
+            one = torch.cat([k[:, :, m].reshape(-1, kv_heads * dim), v], -1)
+            a.append(window_attention(
+                q.view(T, heads, 2, dim)[:, :, m], one, heads, kv_heads, dim, vdim,
+                False, block_tables, block_size, cu, positions, scale, window,
+                keep_first, None, None, None, torch.float32).view(T, heads, vdim))
+        out = a[0] - lam * a[1]
+        out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps) * (1.0 - diff)
+        if gate is not None:
+            out = out * torch.sigmoid(gate.float().reshape(T, heads, -1))
+        return out.reshape(T, heads * vdim).to(out_dtype)
     nk = kv_heads * dim
     out = torch.zeros(T, heads, vdim, dtype=torch.float32, device=q.device)
     cu_l, pos_l = cu.tolist(), positions.tolist()
@@ -564,7 +629,7 @@ def window_attention(q, cache, heads, kv_heads, dim, vdim, whole_key,
         s = s.masked_fill(~ok[None], float("-inf"))
         out[a:e] = torch.einsum("htj,jhd->thd", torch.softmax(s, -1), v)
     if gate is not None:
-        out = out * torch.sigmoid(gate.float())[:, :, None]
+        out = out * torch.sigmoid(gate.float().reshape(T, heads, -1))
     return out.reshape(T, heads * vdim).to(out_dtype)
 
 
@@ -603,3 +668,64 @@ def moe_experts_scaled_input(h, idx, wts, exp_gu, exp_down):
             act = (g * torch.sigmoid(g) * gu[:, ff:]).to(h.dtype)
             out[rows] += F.linear(act, exp_down[e]).float()
     return out
+
+
+def gelu_glu(gu):
+    """gu [T, 2ff] = [gate | up]: gelu_tanh(gate) * up, in gu's dtype."""
+    ff = gu.shape[1] // 2
+    return (gelu_tanh(gu[:, :ff].float()) * gu[:, ff:].float()).to(gu.dtype)
+
+
+def cap_logits(z, scale, cap):
+    """fp32 scale * z, then with ``cap`` > 0 cap * tanh(./cap)."""
+    z = z.float() * scale
+    return cap * torch.tanh(z / cap) if cap > 0 else z
+
+
+# --------------------------------------------------- hyper-connection streams
+
+def row_norm(u, w, eps, center):
+    """Plain-weight norm of fp32 rows: RMS, or with ``center`` the layer norm
+    (mean taken off first)."""
+    if center:
+        u = u - u.mean(-1, keepdim=True)
+    return u * torch.rsqrt(u.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+
+
+def hyper_start(embed, tokens, scale, streams, read_w, norm_w, eps, out_dtype,
+                center):
+    """All streams equal to scale * embed[token]: (x fp32 [T, S, D], the
+    first sublayer's input norm(sum_s read_w[s] x_s) in ``out_dtype``)."""
+    e = embed[tokens].float() * scale
+    x = e[:, None].repeat(1, streams, 1)
+    u = (read_w.float()[None, :, None] * x).sum(1)
+    return x, row_norm(u, norm_w, eps, center).to(out_dtype)
+
+
+def hyper_residual_norm(x, y, y2, y_w, y2_w, y_scale, y2_scale, mix, out_w,
+                        read_w, norm_w, eps, out_dtype, center):
+    """Sublayer tail of the hyper-connection block, in place on the streams
+    x fp32 [T, S, D]: s = y_scale y (+ y2_scale y2), each addend RMS-normed
+    over the width first where a weight (``y_w``/``y2_w``) is given;
+    x_t <- sum_s mix[s, t] x_s + out_w[t] s. With ``norm_w`` returns the next
+    sublayer's input norm(sum_s read_w[s] x_s) in ``out_dtype``, else None."""
+    def side(v, w, a):
+        v = v.float()
+        if w is not None:
+            v = v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+        return a * v
+
+    s = side(y, y_w, y_scale)
+    if y2 is not None:
+        s = s + side(y2, y2_w, y2_scale)
+    new = torch.einsum("nsd,st->ntd", x, mix.float())
+    x.copy_(new + out_w.float()[None, :, None] * s[:, None])
+    if norm_w is None:
+        return None
+    u = (read_w.float()[None, :, None] * x).sum(1)
+    return row_norm(u, norm_w, eps, center).to(out_dtype)
+
+
+def hyper_close_norm(x, rows, norm_w, eps, out_dtype, center):
+    """norm(sum of the streams) of the given rows."""
+    return row_norm(x[rows].sum(1), norm_w, eps, center).to(out_dtype)

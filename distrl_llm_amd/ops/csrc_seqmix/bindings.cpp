@@ -62,7 +62,13 @@ torch::Tensor qk_prepare_kv_write(torch::Tensor proj, int64_t heads, int64_t kv_
                                   c10::optional<torch::Tensor> k_norm_w, double eps,
                                   torch::Tensor positions, c10::optional<torch::Tensor> freqs,
                                   double mag, c10::optional<torch::Tensor> mix,
-                                  torch::Tensor page_slot, torch::Tensor cache);
+                                  torch::Tensor page_slot, torch::Tensor cache, int64_t maps,
+                                  bool unit, double temp_coef, double temp_every,
+                                  c10::optional<torch::Tensor> conv_w,
+                                  c10::optional<torch::Tensor> tails,
+                                  c10::optional<torch::Tensor> cu,
+                                  c10::optional<torch::Tensor> tok_seq,
+                                  c10::optional<torch::Tensor> slots);
 torch::Tensor window_attention(torch::Tensor q, torch::Tensor cache, int64_t heads,
                                int64_t kv_heads, int64_t dim, int64_t vdim, bool whole_key,
                                torch::Tensor block_tables, int64_t block_size,
@@ -70,7 +76,21 @@ torch::Tensor window_attention(torch::Tensor q, torch::Tensor cache, int64_t hea
                                int64_t window, int64_t keep_first,
                                c10::optional<torch::Tensor> r1, c10::optional<torch::Tensor> r2,
                                c10::optional<torch::Tensor> gate,
-                               c10::optional<torch::Tensor> tiles, int64_t max_tile_queries);
+                               c10::optional<torch::Tensor> tiles, int64_t max_tile_queries,
+                               int64_t maps, c10::optional<torch::Tensor> lam_w, double diff,
+                               double eps);
+torch::Tensor gelu_glu(torch::Tensor gu);
+torch::Tensor cap_logits(torch::Tensor z, double scale, double cap);
+std::vector<torch::Tensor> hyper_start(torch::Tensor embed, torch::Tensor tokens, double scale,
+                                       int64_t streams, torch::Tensor read_w, torch::Tensor norm_w,
+                                       double eps, bool out_bf16, bool center);
+c10::optional<torch::Tensor> hyper_residual_norm(
+    torch::Tensor x, torch::Tensor y, c10::optional<torch::Tensor> y2,
+    c10::optional<torch::Tensor> y_w, c10::optional<torch::Tensor> y2_w, double y_scale,
+    double y2_scale, torch::Tensor mix, torch::Tensor out_w, c10::optional<torch::Tensor> read_w,
+    c10::optional<torch::Tensor> norm_w, double eps, bool out_bf16, bool center);
+torch::Tensor hyper_close_norm(torch::Tensor x, torch::Tensor rows, torch::Tensor norm_w, double eps,
+                               bool out_bf16, bool center);
 torch::Tensor capped_glu(torch::Tensor gu, double limit);
 torch::Tensor silu_glu(torch::Tensor gu);
 torch::Tensor qk_norm_kv_write(torch::Tensor proj, int64_t heads, int64_t kv_heads, int64_t dim,
@@ -136,7 +156,13 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("moe_experts_scaled_input", &moe_experts_scaled_input,
         "grouped-GEMM mixture of SiLU-gated experts whose input carries the routing weight");
   m.def("qk_prepare_kv_write", &qk_prepare_kv_write,
-        "q/k norm, half rotary, score-mixing fold of the queries, K/V cache write");
+        "short conv, q/k norm, half rotary, query temperature, score-mixing fold, K/V cache write");
+  m.def("gelu_glu", &gelu_glu, "tanh-GELU-gated GLU activation");
+  m.def("cap_logits", &cap_logits, "scaled, tanh-capped fp32 logits");
+  m.def("hyper_start", &hyper_start, "embedding into residual streams + first norm");
+  m.def("hyper_residual_norm", &hyper_residual_norm,
+        "stream update of a sublayer's output + next read sum and norm");
+  m.def("hyper_close_norm", &hyper_close_norm, "norm of the streams' sum");
   m.def("window_attention", &window_attention,
-        "paged GQA softmax attention: window with kept first tokens, log distance bias, output gate");
+        "paged GQA softmax attention: window with kept first tokens, log distance bias, two maps, output gate");
 }

@@ -3,8 +3,8 @@
 // parallel-residual update (alone, and fused with the next layer's norm),
 // the sandwich residual update (closing norm of a sublayer, residual sum and
 // the next opening norm in one pass; without a closing norm it is the
-// pre-norm tail), the clamped GLU and tanh-GELU activations. Norms may be
-// taken over equal consecutive groups of the row. One workgroup per token row
+// pre-norm tail), the GLU and tanh-GELU activations, the tanh cap of the
+// logits. Norms may be taken over equal consecutive groups of the row. One workgroup per token row
 // for the row-wise ops.
 #include <torch/extension.h>
 #include <ATen/cuda/CUDAContext.h>
@@ -211,26 +211,49 @@ __global__ __launch_bounds__(256) void sandwich_residual_kernel(
 }
 
 // 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))), fp32 inside.
+SM_INLINE float gelu_tanh_f(float z) {
+  return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
 template <typename T>
 __global__ __launch_bounds__(256) void gelu_tanh_kernel(const T* __restrict__ x, int64_t n,
                                                         T* __restrict__ out) {
   const int64_t id = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (id >= n) return;
-  const float z = to_f(x[id]);
-  out[id] = from_f<T>(0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))));
+  out[id] = from_f<T>(gelu_tanh_f(to_f(x[id])));
 }
 
-// gu rows = [gate (ff) | up (ff)]: g = min(gate, limit), u = clamp(up, +-limit),
-// out = g * sigmoid(1.702 g) * (u + 1); SILU: out = gate * sigmoid(gate) * up.
-template <typename T, bool SILU>
-__global__ __launch_bounds__(256) void capped_glu_kernel(
+// gu rows = [gate (ff) | up (ff)]. ACT 0: g = min(gate, limit), u = clamp(up,
+// +-limit), out = g * sigmoid(1.702 g) * (u + 1); 1: silu(gate) * up; 2:
+// gelu_tanh(gate) * up. VEC neighbouring entries per thread (16-byte pieces).
+template <typename T, int ACT, int VEC>
+__global__ __launch_bounds__(256) void glu_kernel(
     const T* __restrict__ gu, int64_t n, int ff, float limit, T* __restrict__ out) {
-  const int64_t id = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+  const int64_t id = ((int64_t)blockIdx.x * blockDim.x + threadIdx.x) * VEC;
   if (id >= n) return;
   const int64_t t = id / ff;
-  const int f = id % ff;
-  const float g = to_f(gu[t * 2 * ff + f]), u = to_f(gu[t * 2 * ff + ff + f]);
-  out[id] = from_f<T>(SILU ? g * sm_sigmoid(g) * u : sm_capped_glu(g, u, limit));
+  const int f = (int)(id - t * ff);
+  struct alignas(VEC * sizeof(T)) piece { T v[VEC]; };
+  const piece gp = *reinterpret_cast<const piece*>(gu + t * 2 * ff + f);
+  const piece up = *reinterpret_cast<const piece*>(gu + t * 2 * ff + ff + f);
+  piece o;
+  #pragma unroll
+  for (int k = 0; k < VEC; ++k) {
+    const float g = to_f(gp.v[k]), u = to_f(up.v[k]);
+    o.v[k] = from_f<T>(ACT == 0 ? sm_capped_glu(g, u, limit)
+                                : (ACT == 1 ? g * sm_sigmoid(g) : gelu_tanh_f(g)) * u);
+  }
+  *reinterpret_cast<piece*>(out + id) = o;
+}
+
+// out = scale * z, then (cap > 0) cap * tanh(./cap); fp32 out.
+template <typename T>
+__global__ __launch_bounds__(256) void cap_logits_kernel(const T* __restrict__ z, int64_t n,
+                                                         float scale, float cap,
+                                                         float* __restrict__ out) {
+  const int64_t id = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (id >= n) return;
+  const float v = to_f(z[id]) * scale;
+  out[id] = cap > 0.f ? cap * tanhf(v / cap) : v;
 }
 
 }  // namespace
@@ -363,6 +386,25 @@ torch::Tensor causal_tap_conv(torch::Tensor h, torch::Tensor w, torch::Tensor ta
   return out;
 }
 
+// Advance the tails of a step's rows to the last taps - 1 inputs (x rows may
+// be a column slice of a wider matrix; C leading columns are taken).
+void tap_tail_update(const torch::Tensor& x, int C, torch::Tensor& tails, const torch::Tensor& cu,
+                     const torch::Tensor& slots, int taps) {
+  if (taps <= 1 || x.size(0) == 0) return;
+  TORCH_CHECK(taps - 1 <= SM_MAX_TAILS, "tap conv: too many taps");
+  auto stream = at::cuda::getCurrentCUDAStream();
+  dim3 g(slots.numel(), SM_CDIV(C, 256));
+  if (x.scalar_type() == at::kBFloat16)
+    tap_tail_kernel<bf16_t><<<g, 256, 0, stream>>>(
+        reinterpret_cast<const bf16_t*>(x.data_ptr()), x.stride(0), tails.data_ptr<float>(),
+        cu.data_ptr<int>(), slots.data_ptr<int>(), C, taps);
+  else
+    tap_tail_kernel<float><<<g, 256, 0, stream>>>(x.data_ptr<float>(), x.stride(0),
+                                                  tails.data_ptr<float>(), cu.data_ptr<int>(),
+                                                  slots.data_ptr<int>(), C, taps);
+  SM_CHECK_LAUNCH();
+}
+
 torch::Tensor tap_conv_silu(torch::Tensor x, torch::Tensor w, torch::Tensor tails,
                             torch::Tensor cu, torch::Tensor tok_seq,
                             torch::Tensor slots, bool out_bf16) {
@@ -481,7 +523,7 @@ c10::optional<torch::Tensor> sandwich_residual_norm(
   return h;
 }
 
-template <bool SILU>
+template <int ACT>
 static torch::Tensor glu_impl(torch::Tensor gu, double limit) {
   SM_CHECK_CUDA(gu);
   TORCH_CHECK(gu.dim() == 2 && gu.size(1) % 2 == 0, "glu: rows are [gate | up]");
@@ -491,21 +533,41 @@ static torch::Tensor glu_impl(torch::Tensor gu, double limit) {
   const int64_t n = T * ff;
   if (n == 0) return out;
   auto stream = at::cuda::getCurrentCUDAStream();
-  if (gu.scalar_type() == at::kBFloat16)
-    capped_glu_kernel<bf16_t, SILU><<<SM_CDIV(n, 256), 256, 0, stream>>>(
-        reinterpret_cast<const bf16_t*>(gu.data_ptr()), n, ff, (float)limit,
-        reinterpret_cast<bf16_t*>(out.data_ptr()));
-  else {
-    SM_CHECK_F32(gu);
-    capped_glu_kernel<float, SILU><<<SM_CDIV(n, 256), 256, 0, stream>>>(
-        gu.data_ptr<float>(), n, ff, (float)limit, out.data_ptr<float>());
-  }
+  const bool bf16 = gu.scalar_type() == at::kBFloat16;
+  if (!bf16) SM_CHECK_F32(gu);
+#define GLU_LAUNCH(TY, VEC)                                                              \
+  glu_kernel<TY, ACT, VEC><<<SM_CDIV(n, 256 * VEC), 256, 0, stream>>>(                   \
+      reinterpret_cast<const TY*>(gu.data_ptr()), n, ff, (float)limit,                   \
+      reinterpret_cast<TY*>(out.data_ptr()))
+  if (bf16) { if (ff % 8 == 0) GLU_LAUNCH(bf16_t, 8); else GLU_LAUNCH(bf16_t, 1); }
+  else { if (ff % 4 == 0) GLU_LAUNCH(float, 4); else GLU_LAUNCH(float, 1); }
+#undef GLU_LAUNCH
   SM_CHECK_LAUNCH();
   return out;
 }
 
-torch::Tensor capped_glu(torch::Tensor gu, double limit) { return glu_impl<false>(gu, limit); }
-torch::Tensor silu_glu(torch::Tensor gu) { return glu_impl<true>(gu, 0.0); }
+torch::Tensor capped_glu(torch::Tensor gu, double limit) { return glu_impl<0>(gu, limit); }
+torch::Tensor silu_glu(torch::Tensor gu) { return glu_impl<1>(gu, 0.0); }
+torch::Tensor gelu_glu(torch::Tensor gu) { return glu_impl<2>(gu, 0.0); }
+
+torch::Tensor cap_logits(torch::Tensor z, double scale, double cap) {
+  SM_CHECK_CUDA(z);
+  auto out = torch::empty(z.sizes(), z.options().dtype(at::kFloat));
+  const int64_t n = z.numel();
+  if (n == 0) return out;
+  auto stream = at::cuda::getCurrentCUDAStream();
+  if (z.scalar_type() == at::kBFloat16)
+    cap_logits_kernel<bf16_t><<<SM_CDIV(n, 256), 256, 0, stream>>>(
+        reinterpret_cast<const bf16_t*>(z.data_ptr()), n, (float)scale, (float)cap,
+        out.data_ptr<float>());
+  else {
+    SM_CHECK_F32(z);
+    cap_logits_kernel<float><<<SM_CDIV(n, 256), 256, 0, stream>>>(
+        z.data_ptr<float>(), n, (float)scale, (float)cap, out.data_ptr<float>());
+  }
+  SM_CHECK_LAUNCH();
+  return out;
+}
 
 torch::Tensor gelu_tanh(torch::Tensor x) {
   SM_CHECK_CUDA(x);

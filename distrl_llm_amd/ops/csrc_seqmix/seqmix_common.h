@@ -59,6 +59,21 @@ SM_INLINE float sm_block_sum(float x, float* red) {
   return r;
 }
 SM_INLINE float sm_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+// Differential attention: lam_w = lq1 | lk1 | lq2 | lk2 (dk entries each);
+// lambda = exp(lq1.lk1) - exp(lq2.lk2) + diff, the difference's norm takes eps.
+struct wa_diff {
+  const float* lam_w;
+  float diff, eps;
+};
+// Every lane of the wave takes part and gets lambda.
+SM_INLINE float wa_lambda(const wa_diff& df, int dk, int lane) {
+  float s1 = 0.f, s2 = 0.f;
+  for (int k = lane; k < dk; k += SM_WAVE) {
+    s1 = fmaf(df.lam_w[k], df.lam_w[dk + k], s1);
+    s2 = fmaf(df.lam_w[2 * dk + k], df.lam_w[3 * dk + k], s2);
+  }
+  return expf(sm_wave_sum(s1)) - expf(sm_wave_sum(s2)) + df.diff;
+}
 // clamped GLU: g = min(gate, limit), u = clamp(up, +-limit), g sigmoid(1.702 g) (u + 1)
 SM_INLINE float sm_capped_glu(float g, float u, float limit) {
   g = fminf(g, limit);

@@ -1,6 +1,6 @@
 """Prefill and decode throughput of the layer-list designs (Nibalix,
-Nedasun, Kakilorn, Legilix) beside one another and beside the dense transformer of equal size
-(``bench.py --hybrid-bench``).
+Nedasun, Kakilorn, Legilix, Sagedra) beside one another and beside the dense
+transformer of equal size (``bench.py --hybrid-bench``).
 
 All models get random weights at layer sizes that resemble a real model
 and run through their own engine's ``generate`` — scheduler, cache, step
@@ -148,13 +148,48 @@ def legilix_bench_config(s: dict) -> dict:
             "width": s["width"]}
 
 
+def sagedra_bench_config(s: dict) -> dict:
+    """Same width, head count and value size as the other designs of the
+    size, 4 query heads per kv head, four residual streams. Six layers run as
+    eight (layers 1 and 2 twice): differential attention (two maps of 64 over
+    values of 128, full causal, 3 taps) and pairs of windowed attention
+    (128/128, window of the size) beside the delta rule with half the heads;
+    dense feed-forwards as wide as the experts one token uses elsewhere."""
+    kvh = max(1, s["heads"] // 4)
+    dense = {"kind": "dense", "ff": s["top"] * s["ff"]}
+    attention = {"heads": s["heads"], "kv_heads": kvh, "dim": 64, "vdim": 128,
+                 "scale": 64 ** -0.5, "conv": 3, "diff": 0.5,
+                 "q_temp": {"coef": 0.1, "every": 4096}}
+    left = {"heads": s["heads"], "kv_heads": kvh, "dim": 128, "vdim": 128,
+            "scale": 128 ** -0.5, "mask": {"size": s["window"]},
+            "rot": {"base": 500000.0, "dims": 128,
+                    "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0,
+                                "original": 8192}}}
+    right = {"heads": s["heads"] // 2, "kv_heads": max(1, kvh // 2), "dim": 128,
+             "vdim": 128, "conv": 4}
+    layers = []
+    for i in range(s["layers"] - 2):
+        if i % 3 == 2:
+            layers.append({"type": "parallel", "mixer": {"left": left, "right": right},
+                           "mlp": dense})
+        else:
+            layers.append({"type": "attention", "mixer": attention, "mlp": dense})
+    return {"architecture": "Sagedra", "embedding": {"scale": 1.0}, "layers": layers,
+            "logit_softcap": 30.0, "loop": {"start": 1, "stop": 3, "times": 2},
+            "norm": {"eps": 1e-5}, "streams": 4, "vocab": s["vocab"],
+            "width": s["width"]}
+
+
 def _build_hybrid(s, device, max_len, batch, design="nibalix"):
     from .engine.hybrid_engine import HybridEngine
     from .models.hybrid import (HybridLM, kakilorn_spec_from_config,
                                 legilix_spec_from_config,
                                 nedasun_spec_from_config,
-                                nibalix_spec_from_config)
-    if design == "legilix":
+                                nibalix_spec_from_config,
+                                sagedra_spec_from_config)
+    if design == "sagedra":
+        spec = sagedra_spec_from_config(sagedra_bench_config(s))
+    elif design == "legilix":
         spec = legilix_spec_from_config(legilix_bench_config(s))
     elif design == "kakilorn":
         spec = kakilorn_spec_from_config(kakilorn_bench_config(s))
@@ -208,7 +243,8 @@ def measure(engine, vocab, batch, prompt_len, new_tokens, device):
             "prefill_s": t_pre, "decode_ms_per_step": 1e3 * dec / (new_tokens - 1)}
 
 
-def run(sizes, device, batch=16, prompt_len=1024, new_tokens=33, which=("legilix", "kakilorn", "nedasun", "nibalix", "dense")):
+def run(sizes, device, batch=16, prompt_len=1024, new_tokens=33,
+        which=("sagedra", "legilix", "kakilorn", "nedasun", "nibalix", "dense")):
     out = []
     for name in sizes:
         s = SIZES[name]

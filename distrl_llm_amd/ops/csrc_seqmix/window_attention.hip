@@ -81,7 +81,9 @@ template <> struct wa_vec<float> {
 // [H, G dk]. CONV: every q/k/v channel is first convolved over its sequence
 // (inputs before the portion come from tails[slot]); step: every row of the
 // batch holds one token, and the thread that convolves a channel advances its
-// tail. PAIR: dk and nv are even and rows start on 4-byte borders, so entries
+// tail. TAPS: 0 no convolution, 2 .. 4 that many taps, unrolled (a token whose
+// history lies in the portion issues all its loads at once), -1 any number.
+// PAIR: dk and nv are even and rows start on 4-byte borders, so entries
 // go two at a time.
 struct qkp_conv {
   const float* w;        // [C, taps]
@@ -91,7 +93,7 @@ struct qkp_conv {
   const int* slots;
   int taps, step;
 };
-template <typename T, bool PAIR, bool CONV>
+template <typename T, bool PAIR, int TAPS>
 __global__ __launch_bounds__(256) void qk_prepare_kv_write_kernel(
     const T* __restrict__ proj, int64_t ldp, int H, int G, int dk, int nv,
     const float* __restrict__ qw, const float* __restrict__ kw, float eps,
@@ -105,7 +107,8 @@ __global__ __launch_bounds__(256) void qk_prepare_kv_write_kernel(
   const int64_t t = blockIdx.x;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const T* row = proj + t * ldp;
-  const int C = nqk + nv, keep = CONV ? cv.taps - 1 : 0;
+  constexpr bool CONV = TAPS != 0;
+  const int C = nqk + nv, keep = TAPS > 0 ? TAPS - 1 : (CONV ? cv.taps - 1 : 0);
   int rel = 0;
   float* tl = nullptr;
   if (CONV) {
@@ -130,21 +133,38 @@ __global__ __launch_bounds__(256) void qk_prepare_kv_write_kernel(
     return fmaf(w[keep], x, acc);
   };
   auto fetch2 = [&](int i) -> float2 {
-    const float2 x = wa_vec<T>::load2(row + i);
-    if (!CONV) return x;
-    const float* w = cv.w + (int64_t)i * cv.taps;
+    if (!CONV) return wa_vec<T>::load2(row + i);
+    const float* w = cv.w + (int64_t)i * (keep + 1);
     float a0 = 0.f, a1 = 0.f;
+    if constexpr (TAPS > 0) {
+      if (rel >= TAPS - 1 && !cv.step) {             // uniform over the workgroup
+        float2 v[TAPS], wv[TAPS];                    // wv: both channels' weights in a row
+        #pragma unroll
+        for (int j = 0; j < TAPS; ++j) {
+          v[j] = wa_vec<T>::load2(row + (int64_t)(j - (TAPS - 1)) * ldp + i);
+          wv[j] = *reinterpret_cast<const float2*>(w + 2 * j);
+        }
+        const float* wf = reinterpret_cast<const float*>(wv);
+        #pragma unroll
+        for (int j = 0; j < TAPS; ++j) {
+          a0 = fmaf(wf[j], v[j].x, a0);
+          a1 = fmaf(wf[TAPS + j], v[j].y, a1);
+        }
+        return make_float2(a0, a1);
+      }
+    }
+    const float2 x = wa_vec<T>::load2(row + i);
     for (int j = 0; j < keep; ++j) {
       const int src = rel - keep + j;
       const float2 v = (src >= 0)
           ? wa_vec<T>::load2(row + (int64_t)(j - keep) * ldp + i)
           : *reinterpret_cast<const float2*>(tl + (int64_t)(keep + src) * C + i);
       a0 = fmaf(w[j], v.x, a0);
-      a1 = fmaf(w[cv.taps + j], v.y, a1);
+      a1 = fmaf(w[keep + 1 + j], v.y, a1);
       if (cv.step && j > 0) *reinterpret_cast<float2*>(tl + (int64_t)(j - 1) * C + i) = v;
     }
     if (cv.step && keep > 0) *reinterpret_cast<float2*>(tl + (int64_t)(keep - 1) * C + i) = x;
-    return make_float2(fmaf(w[keep], x.x, a0), fmaf(w[cv.taps + keep], x.y, a1));
+    return make_float2(fmaf(w[keep], x.x, a0), fmaf(w[2 * keep + 1], x.y, a1));
   };
   if (PAIR) {
     for (int i = 2 * threadIdx.x; i < nqk; i += 2 * blockDim.x) {
@@ -837,9 +857,9 @@ torch::Tensor qk_prepare_kv_write(torch::Tensor proj, int64_t heads, int64_t kv_
   const int64_t esz = is_bf16 ? 2 : 4;
   const bool pair = dk % 2 == 0 && nv % 2 == 0 && proj.stride(0) % 2 == 0 &&
                     reinterpret_cast<uintptr_t>(proj.data_ptr()) % (2 * esz) == 0;
-#define QKP_LAUNCH(TY, PAIRV, CONVV)                                                           \
+#define QKP_LAUNCH(TY, PAIRV, TAPSV)                                                           \
   do {                                                                                         \
-    auto kern = qk_prepare_kv_write_kernel<TY, PAIRV, CONVV>;                                  \
+    auto kern = qk_prepare_kv_write_kernel<TY, PAIRV, TAPSV>;                                  \
     static int raised = 0;     /* per variant; not repeated under graph capture */             \
     if (lds > 64 * 1024 && (int)lds > raised) {                                                \
       TORCH_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(kern),                     \
@@ -856,8 +876,11 @@ torch::Tensor qk_prepare_kv_write(torch::Tensor proj, int64_t heads, int64_t kv_
   } while (0)
 #define QKP_BY_CONV(TY, PAIRV)                            \
   do {                                                    \
-    if (cv.w != nullptr) QKP_LAUNCH(TY, PAIRV, true);     \
-    else QKP_LAUNCH(TY, PAIRV, false);                    \
+    if (cv.w == nullptr) QKP_LAUNCH(TY, PAIRV, 0);        \
+    else if (PAIRV && cv.taps == 2) QKP_LAUNCH(TY, PAIRV, 2); \
+    else if (PAIRV && cv.taps == 3) QKP_LAUNCH(TY, PAIRV, 3); \
+    else if (PAIRV && cv.taps == 4) QKP_LAUNCH(TY, PAIRV, 4); \
+    else QKP_LAUNCH(TY, PAIRV, -1);                       \
   } while (0)
   if (is_bf16) { if (pair) QKP_BY_CONV(bf16_t, true); else QKP_BY_CONV(bf16_t, false); }
   else { if (pair) QKP_BY_CONV(float, true); else QKP_BY_CONV(float, false); }

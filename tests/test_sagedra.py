@@ -196,7 +196,8 @@ def test_rotary_table():
 @pytest.mark.parametrize("H,G,dk,dv,maps,rot_dims,unit,temp,taps", [
     (4, 2, 6, 10, 2, 0, False, True, 3), (3, 3, 8, 5, 1, 6, True, False, 0),
     (6, 2, 5, 3, 2, 0, False, True, 4), (2, 1, 72, 4, 1, 70, True, True, 2),
-    (1, 1, 2, 1, 2, 2, True, False, 1), (5, 1, 4, 6, 2, 0, False, False, 5)])
+    (1, 1, 2, 1, 2, 2, True, False, 1), (5, 1, 4, 6, 2, 0, False, False, 5),
+    (2, 1, 8, 6, 2, 0, False, True, 4)])
 def test_prepare(dev, H, G, dk, dv, maps, rot_dims, unit, temp, taps):
     """Convolution with carried tails, rotation, norm after it, query
     temperature and page write: two rows of a step cut into portions down to

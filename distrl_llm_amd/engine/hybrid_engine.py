@@ -25,7 +25,8 @@ import torch.nn.functional as F
 
 from ..config import EngineConfig, SamplingParams
 from ..models.hybrid import (DeltaRuleSpec, GluSpec, HybridLM,
-                             LatentAttentionSpec, MlpSpec, ParallelMixerSpec,
+                             LatentAttentionSpec, LinearAttentionSpec,
+                             LinearUnitSpec, MlpSpec, ParallelMixerSpec,
                              SigmoidAttentionSpec, SinkAttentionSpec,
                              WindowAttentionSpec)
 from ..ops import functional as OF
@@ -78,7 +79,7 @@ class _DecodeGraph:
                     block_tables=tables + [[scratch]] * pad,
                     tiles=[(b, b, 1) for b in range(self.rows)], max_tile=1,
                     wide_tiles=[(b, b, 1) for b in range(self.rows)],
-                    max_wide_tile=1)
+                    max_wide_tile=1, wide_cu=list(range(self.rows + 1)))
         return eng._pack(tokens + [0] * pad, meta, list(range(self.rows)),
                          max_nb=self.max_nb)
 
@@ -230,12 +231,15 @@ class HybridEngine:
         lengths = [len(t) for _, t in work]
         tiles, max_tile = SM.query_tiles(lengths)
         wide, max_wide = SM.query_tiles(lengths, SM.WIDE_QUERY_TILE)
+        wide_cu = [0]
+        for n in lengths:
+            wide_cu.append(wide_cu[-1] + -(-n // SM.WIDE_QUERY_TILE))
         chunks, chunk_cu = SM.scan_chunks(lengths)
         meta = dict(positions=positions, tok_seq=tok_seq, page_slot=page_slot,
                     cu=cu, slots=slot_idx,
                     block_tables=[q.block_table for q, _ in work],
                     tiles=tiles, max_tile=max_tile, wide_tiles=wide,
-                    max_wide_tile=max_wide, scan_chunks=chunks,
+                    max_wide_tile=max_wide, wide_cu=wide_cu, scan_chunks=chunks,
                     scan_cu=chunk_cu)
         return tokens, meta, want_rows
 
@@ -256,6 +260,7 @@ class HybridEngine:
                            ("tiles", tiles),
                            ("wide_tiles", [v for t in meta.get("wide_tiles", [])
                                            for v in t]),
+                           ("wide_cu", meta.get("wide_cu", [])),
                            ("want", want_rows),
                            ("scan_chunks", [v for c in meta.get("scan_chunks", [])
                                             for v in c]),
@@ -276,6 +281,7 @@ class HybridEngine:
         meta["block_tables"] = cut("block_tables").view(-1, lay["max_nb"])
         meta["tiles"] = cut("tiles").view(-1, 3)
         meta["wide_tiles"] = cut("wide_tiles").view(-1, 3)
+        meta["wide_cu"] = cut("wide_cu")
         meta["max_wide_tile"] = lay["max_wide_tile"]
         meta["scan_chunks"] = cut("scan_chunks").view(-1, 3)
         meta["scan_cu"] = cut("scan_cu")
@@ -445,7 +451,8 @@ class HybridEngine:
             L.dist_r2 if m.log_distance else None, gate, self.dtype,
             tiles=meta["wide_tiles"], max_tile=meta["max_wide_tile"],
             maps=m.maps, lam_w=L.lam_w if m.maps == 2 else None, diff=m.diff,
-            eps=self.spec.norm_eps)
+            eps=self.spec.norm_eps, chunk=m.chunk, softcap=m.softcap,
+            sink=L.sink if m.sink else None)
         return F.linear(o, L.out_w, L.out_b if m.out_bias else None)
 
     def _mix_delta(self, i, m, L, hm, meta, proj=None, x32=None):
@@ -478,6 +485,27 @@ class HybridEngine:
                                 gate_sigmoid=(m.gate == "sigmoid"), **own)
         return F.linear(o, L.out_w)
 
+    def _mix_linear_attention(self, i, m, L, hm, meta, proj=None, x32=None):
+        if proj is None:
+            proj = F.linear(hm, L.in_w)
+        powers = self._const(("decay", i),
+                             lambda: SM.decay_powers(m.decay, self.device))
+        o = SM.linear_attention(proj, m.heads, m.dim, m.vdim, powers, L.onorm_w,
+                                self.spec.norm_eps, self.slots.recurrent[i],
+                                meta["cu"], meta["slots"], self.dtype,
+                                max_tile=meta["max_wide_tile"])
+        return F.linear(o, L.out_w)
+
+    def _mix_linear_unit(self, i, m, L, hm, meta, proj=None, x32=None):
+        if proj is None:
+            proj = F.linear(hm, L.in_w, L.in_b)
+        o = SM.linear_unit(proj, L.conv_w, L.conv_b, self.slots.mixer_tails[i],
+                           L.gates_w, L.gates_b, L.lam, m.c,
+                           self.slots.recurrent[i], meta["cu"], meta["tok_seq"],
+                           meta["slots"], self.dtype, tiles=meta["wide_tiles"],
+                           tile_cu=meta["wide_cu"])
+        return F.linear(o, L.out_w)
+
     def _mix_unit(self, key, m, W, hm, meta, shared, proj=None, x32=None):
         if isinstance(m, LatentAttentionSpec):
             return self._mix_latent(key, m, W, hm, meta, proj, x32)
@@ -489,13 +517,17 @@ class HybridEngine:
             return self._mix_window_attention(key, m, W, hm, meta, proj, x32)
         if isinstance(m, DeltaRuleSpec):
             return self._mix_delta(key, m, W, hm, meta, proj, x32)
+        if isinstance(m, LinearAttentionSpec):
+            return self._mix_linear_attention(key, m, W, hm, meta, proj, x32)
+        if isinstance(m, LinearUnitSpec):
+            return self._mix_linear_unit(key, m, W, hm, meta, proj, x32)
         return self._mix_mingru(key, m, W, hm, meta, proj, x32)
 
     def _mixer(self, i, ls, L, hm, meta, shared, x32=None):
         """-> (output, second output or None, their scales)."""
         m = ls.mixer
         if isinstance(m, ParallelMixerSpec):
-            proj = F.linear(hm, L.in_w)
+            proj = F.linear(hm, L.in_w, L.in_b if m.in_bias else None)
             nl = m.left.in_size
             left = self._mix_unit((i, 0), m.left, L.left, hm, meta, shared,
                                   proj[:, :nl], x32)
@@ -522,8 +554,12 @@ class HybridEngine:
                                                    L.exp_down), None
             return SM.moe_experts(hb, idx, wts, L.exp_gu, L.exp_down), None
         if f.routing == "all":
-            idx, wts = SM.moe_route_all(hb, L.router_w, L.correction, f.top,
-                                        f.scale)
+            # a correction that no checkpoint fills is not read
+            idx, wts = SM.moe_route_all(hb, L.router_w,
+                                        None if f.expert == "relu2" else L.correction,
+                                        f.top, f.scale, f.groups, f.renorm)
+            if f.expert == "relu2":
+                return SM.moe_experts_relu2(hb, idx, wts, L.exp_gu, L.exp_down), None
             y = SM.moe_experts_glu(hb, idx, wts, L.exp_gu, L.exp_down, f.limit)
             if f.shared is None:
                 return y, None
@@ -544,6 +580,8 @@ class HybridEngine:
             x = self._layers_pre_norm(tokens, meta, capture)
         elif S.block == "hyper":
             x = self._layers_hyper(tokens, meta, capture)
+        elif S.block == "parallel":
+            x = self._layers_parallel(tokens, meta, capture)
         else:
             x = self._layers_parallel_gated(tokens, meta, capture)
         if want_rows.numel() == 0:
@@ -707,6 +745,45 @@ class HybridEngine:
                                             ctr)
             if capture is not None:
                 capture.append(x.sum(1))
+        return x
+
+    def _layers_parallel(self, tokens, meta, capture):
+        """One norm per layer feeds both sublayers, x += mixer(h) + ff(h).
+        Layer tail (norms of a pair's sides, sums, what a pass of a loop adds
+        at its start) and the next layer's norm are one kernel."""
+        S, M, dt = self.spec, self.model, self.dtype
+        eps, off = S.norm_eps, S.norm_offset
+        shared = {}
+        starts = S.pass_starts if S.loop_inject else {}
+
+        def inject(r):
+            t = starts.get(r)
+            if t is None:
+                return None
+            return (M.embed if t > 0 else None, tokens, S.embed_scale, M.loop_step[t])
+
+        first = inject(0)
+        x, hb = SM.parallel_start(M.embed, tokens, S.embed_scale,
+                                  first[3] if first else None,
+                                  M.layers[S.runs[0]].norm_w, eps, dt, off)
+        for i, ls, L, after in self._layer_runs():
+            y, y2, (a, b) = self._mixer(i, ls, L, hb, meta, shared)
+            normed = y2 is not None and ls.mixer.out_norm
+            f = None
+            if ls.mlp is not None:
+                f, f2 = self._ff(ls.mlp, L, hb)
+                if f2 is not None:
+                    f = f.float() + f2.float()
+            nxt, inj = (after.norm_w if after is not None else None), inject(i + 1)
+            tail = (x, y, y2, L.left_norm_w if normed else None,
+                    L.right_norm_w if normed else None, a, b, f)
+            if capture is None:
+                hb = SM.parallel_residual_norm(*tail, inj, nxt, eps, dt, off)
+                continue
+            SM.parallel_residual_norm(*tail, None, None, eps, dt, off)
+            capture.append(x.clone())
+            hb = SM.parallel_residual_norm(x, None, None, None, None, 1.0, 1.0, None,
+                                           inj, nxt, eps, dt, off)
         return x
 
     def score(self, ids: Seq[int]) -> torch.Tensor:

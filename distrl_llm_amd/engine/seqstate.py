@@ -14,10 +14,11 @@ come and go:
   index unless layers are looped), or (run, side) for the two sides of a
   parallel pair.
 * :class:`StateSlotPool` — fixed-size fp32 state per live sequence: the
-  last ``taps - 1`` inputs of every short convolution (the block's own, or
-  a delta-rule or attention layer's over its q/k/v channels) and the state of every
-  recurrent layer (a vector for minGRU, a matrix per head for the delta
-  rule). A slot is zeroed when it is handed out, so whatever its previous
+  last ``taps - 1`` inputs of every short convolution (the block's own, a
+  delta-rule or attention layer's over its q/k/v channels, or a recurrent
+  unit's) and the state of every
+  recurrent layer (a vector for minGRU and the linear recurrent unit, a
+  matrix per head for the delta rule and linear attention). A slot is zeroed when it is handed out, so whatever its previous
   owner left cannot leak.
 """
 
@@ -27,10 +28,9 @@ from typing import Dict, List
 
 import torch
 
-from ..models.hybrid import (DeltaRuleSpec, HybridSpec, LatentAttentionSpec,
-                             MinGRUSpec, SigmoidAttentionSpec,
-                             SinkAttentionSpec, WindowAttentionSpec,
-                             mixer_conv, mixer_units)
+from ..models.hybrid import (HybridSpec, LatentAttentionSpec,
+                             SigmoidAttentionSpec, SinkAttentionSpec,
+                             WindowAttentionSpec, mixer_conv, mixer_units)
 from .kvcache import BlockAllocator
 
 
@@ -93,7 +93,7 @@ class StateSlotPool:
             i: torch.zeros(num_slots + 1, m.state_size, dtype=torch.float32,
                            device=device)
             for i, m in mixer_units(spec)
-            if isinstance(m, (MinGRUSpec, DeltaRuleSpec))}
+            if hasattr(m, "state_size")}
         # a mixer's own short convolution: mixer unit ->
         # [slots + 1, taps - 1, channels] fp32
         self.mixer_tails: Dict[object, torch.Tensor] = {

@@ -88,6 +88,22 @@ parameter, so another design can reuse them in another order.
   rotary with rescaled frequencies, q/k RMS-normed after it, a sigmoid gate
   per output entry) beside the per-head gated delta rule;
 * feed-forward: a dense tanh-GELU GLU.
+
+``Pedazen`` is the sixth:
+
+* residual stream in fp32; one offset-weight RMS norm per layer feeds both
+  sublayers, ``x += mixer(h) + ff(h)`` (parallel arrangement, ungated); a
+  stretch of layers runs several times in a row, every pass starting with a
+  learned vector of its own and, from the second on, the embedding output
+  added to the residual; the embedding table is the output matrix;
+* mixers: linear attention with a fixed decay per head (SiLU on q, k and v,
+  fp32 matrix state, one RMS norm over all heads, sigmoid output gate) and a
+  parallel pair with normed sides: chunked attention (a query sees its own
+  chunk only; q/k RMS-normed, half rotary, capped scores, a per-head sink)
+  beside a real-gated linear recurrent unit (short convolution, block-diagonal
+  gates, fp32 vector state, GELU branch);
+* feed-forward: a dense tanh-GELU GLU, or squared-ReLU experts whose router
+  chooses within the best groups of experts and renormalises the scores.
 """
 
 from __future__ import annotations
@@ -300,7 +316,10 @@ class WindowAttentionSpec:
     output projection, and ``maps`` = 2: differential attention, where every
     head has two query/key maps over the same values and gives
     ``N(a1 - lambda a2) (1 - diff)``, N a weightless RMS norm over the head's
-    values and ``lambda = e^(lq1.lk1) - e^(lq2.lk2) + diff``."""
+    values and ``lambda = e^(lq1.lk1) - e^(lq2.lk2) + diff``; ``chunk``:
+    position i sees only the keys of its own chunk, floor(i / chunk) =
+    floor(j / chunk); ``softcap``: scores become cap tanh(score / cap);
+    ``sink``: a learned per-head term in the softmax denominator."""
     heads: int
     kv_heads: int
     dim: int
@@ -323,8 +342,15 @@ class WindowAttentionSpec:
     out_bias: bool = False
     maps: int = 1
     diff: float = 0.0
+    chunk: int = 0                      # 0 = no chunks
+    softcap: float = 0.0                # 0 = scores are not capped
+    sink: bool = False
 
     kind = "window_attention"
+
+    @property
+    def in_bias(self) -> bool:
+        return self.qkv_bias
 
     @property
     def q_size(self) -> int:           # head by head, map by map
@@ -362,6 +388,64 @@ class WindowAttentionSpec:
 
 
 @dataclass(frozen=True)
+class LinearAttentionSpec:
+    """Linear attention with a fixed decay per head: SiLU on q, k and v,
+    ``S <- decay_h S + k v^T``, ``o = S^T q``; the concatenated heads are
+    RMS-normed together (plain weight) and scaled by a sigmoid gate per
+    entry read from the mixer input."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: tuple            # one factor per head
+
+    kind = "linear_attention"
+
+    @property
+    def q_size(self) -> int:
+        return self.heads * self.dim
+
+    @property
+    def v_size(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def in_size(self) -> int:          # [q | k | v | gate]
+        return 2 * self.q_size + 2 * self.v_size
+
+    @property
+    def state_size(self) -> int:       # per head value-major: S^T
+        return self.heads * self.dim * self.vdim
+
+
+@dataclass(frozen=True)
+class LinearUnitSpec:
+    """Real-gated linear recurrent unit between two branches of size
+    ``width``: y = gelu_tanh(W_y h + b) and u, a short causal convolution
+    (with bias) of W_x h + b. Gates r, i are sigmoids of block-diagonal maps
+    of u (``blocks`` square matrices); with log a = -c r softplus(lam):
+    ``S <- a S + sqrt(1 - a^2) i u``, result S y."""
+    width: int
+    blocks: int
+    taps: int
+    c: float = 8.0
+
+    kind = "linear_unit"
+    in_bias = True
+
+    @property
+    def in_size(self) -> int:          # [y | x]
+        return 2 * self.width
+
+    @property
+    def block_size(self) -> int:
+        return self.width // self.blocks
+
+    @property
+    def state_size(self) -> int:
+        return self.width
+
+
+@dataclass(frozen=True)
 class ParallelMixerSpec:
     """Two mixers that read the same input; the result is
     ``left_scale * left + right_scale * right``, with ``out_norm`` each side
@@ -377,6 +461,10 @@ class ParallelMixerSpec:
     @property
     def in_size(self) -> int:
         return self.left.in_size + self.right.in_size
+
+    @property
+    def in_bias(self) -> bool:
+        return any(getattr(m, "in_bias", False) for m in (self.left, self.right))
 
 
 def mixer_units(spec: "HybridSpec"):
@@ -399,6 +487,8 @@ def mixer_conv(m):
         return m.taps, m.conv_channels
     if isinstance(m, WindowAttentionSpec) and m.conv_taps:
         return m.conv_taps, m.conv_channels
+    if isinstance(m, LinearUnitSpec):
+        return m.taps, m.width
     return None
 
 
@@ -473,6 +563,13 @@ class MoESpec:
     # the weight multiplies the expert's input (expert(w h)) instead of its
     # output
     scale_input: bool = False
+    # (count, keep): experts form ``count`` equal groups of neighbours, only
+    # those of the ``keep`` groups with the largest single scores can be chosen
+    groups: Optional[tuple] = None
+    renorm: bool = False    # weights are divided by their sum (routing "all")
+    # expert "glu": gated pair of input matrices; "relu2": one input matrix,
+    # down(relu(up h)^2)
+    expert: str = "glu"
     identity: int = 0       # trailing router outputs that pass the input through
     scale: float = 1.0
     limit: float = 0.0      # 0: SiLU-gated experts; > 0: clamped GLU experts
@@ -498,6 +595,7 @@ class HybridSpec:
     # "sandwich": norm before and after each sublayer, one after the other;
     # "post_norm": sublayers read the residual, only their output is normed;
     # "pre_norm": x += sublayer(norm(x)), nothing else;
+    # "parallel": one norm feeds mixer and feed-forward, x += mixer(h) + ff(h);
     # "hyper": ``streams`` residual streams, u = sum_s in[s] x_s,
     # x_t <- sum_s mix[s, t] x_s + out[t] sublayer(norm(u))
     block: str = "parallel_gated"
@@ -515,6 +613,9 @@ class HybridSpec:
     # (start, stop, times): layers start .. stop - 1 run ``times`` times in a
     # row, every pass with a cache or state of its own
     loop: Optional[tuple] = None
+    # every pass starts by adding its own learned vector to the residual, and
+    # from the second on the embedding output before it ("parallel" block)
+    loop_inject: bool = False
 
     @property
     def num_layers(self) -> int:
@@ -528,6 +629,14 @@ class HybridSpec:
             return tuple(range(n))
         a, b, times = self.loop
         return (tuple(range(a)) + tuple(range(a, b)) * times + tuple(range(b, n)))
+
+    @property
+    def pass_starts(self) -> dict:
+        """{index of the run that opens a pass of the loop: number of the pass}."""
+        if self.loop is None:
+            return {}
+        a, b, times = self.loop
+        return {a + t * (b - a): t for t in range(times)} if b > a else {}
 
 
 def nibalix_spec_from_config(cfg: dict, name: str = "nibalix") -> HybridSpec:
@@ -625,6 +734,8 @@ def _make_mixer_weights(mod, m, D, P, packed_input=True):
     f32 = torch.float32
     if packed_input:
         mod.in_w = P(m.in_size if hasattr(m, "in_size") else 3 * m.width, D)
+        if getattr(m, "in_bias", False):    # added by the projection GEMM
+            mod.in_b = P(m.in_size)
     if isinstance(m, LatentAttentionSpec):
         if m.kv_from is None:
             mod.latent_norm_w = P(m.kv_rank, dt=f32)
@@ -646,10 +757,10 @@ def _make_mixer_weights(mod, m, D, P, packed_input=True):
         mod.pos_bias = P(m.heads, dt=f32)
         mod.out_w = P(D, m.heads * m.vdim)
     elif isinstance(m, WindowAttentionSpec):
-        if m.qkv_bias:                  # added by the projection GEMM
-            mod.in_b = P(m.in_size)
         if m.qk_norm:
             mod.q_norm_w, mod.k_norm_w = P(m.dim, dt=f32), P(m.dim, dt=f32)
+        if m.sink:
+            mod.sink = P(m.heads, dt=f32)
         if m.score_mix:
             mod.talk = P(m.heads, m.heads, dt=f32)
         if m.log_distance:
@@ -674,6 +785,17 @@ def _make_mixer_weights(mod, m, D, P, packed_input=True):
             mod.gate_up = P(m.v_size, m.gate_rank)
         mod.onorm_w = P(m.vdim, dt=f32)
         mod.out_w = P(D, m.v_size)
+    elif isinstance(m, LinearAttentionSpec):
+        mod.onorm_w = P(m.v_size, dt=f32)
+        mod.out_w = P(D, m.v_size)
+    elif isinstance(m, LinearUnitSpec):
+        n = m.block_size
+        mod.conv_w, mod.conv_b = P(m.width, m.taps, dt=f32), P(m.width, dt=f32)
+        # [gate r; gate i] of every block
+        mod.gates_w = P(2, m.blocks, n, n)
+        mod.gates_b = P(2, m.width, dt=f32)
+        mod.lam = P(m.width, dt=f32)
+        mod.out_w = P(D, m.width)
     else:
         mod.in_b = P(3 * m.width, dt=f32)
         mod.out_w = P(D, m.width)
@@ -698,7 +820,9 @@ class HybridLayer(nn.Module):
                                 requires_grad=False)
 
         f32 = torch.float32
-        if spec.block == "post_norm":
+        if spec.block == "parallel":
+            self.norm_w = P(D, dt=f32)
+        elif spec.block == "post_norm":
             self.post_w = P(D, dt=f32)
             if ls.mlp is not None:
                 self.ff_post_w = P(D, dt=f32)
@@ -731,6 +855,8 @@ class HybridLayer(nn.Module):
         if isinstance(m, ParallelMixerSpec):
             # both sides read one packed projection of the shared input
             self.in_w = P(m.in_size, D)
+            if m.in_bias:
+                self.in_b = P(m.in_size)
             self.left, self.right = nn.Module(), nn.Module()
             _make_mixer_weights(self.left, m.left, D, P, packed_input=False)
             _make_mixer_weights(self.right, m.right, D, P, packed_input=False)
@@ -750,7 +876,7 @@ class HybridLayer(nn.Module):
                 self.router_b = P(n, dt=f32)
             if f.routing == "all":
                 self.correction = P(n, dt=f32)
-            self.exp_gu = P(f.experts, 2 * f.ff, D)
+            self.exp_gu = P(f.experts, f.ff if f.expert == "relu2" else 2 * f.ff, D)
             self.exp_down = P(f.experts, D, f.ff)
             if f.shared is not None:
                 self.shared_gu = P(2 * f.shared.ff, D)
@@ -779,6 +905,8 @@ class HybridLM(nn.Module):
         self.final_norm_w = P(D, dt=f32)
         # a tied output matrix is the embedding parameter itself
         self.head = self.embed if spec.tied_head else P(spec.vocab_size, D)
+        if spec.loop_inject and spec.loop is not None:
+            self.loop_step = P(spec.loop[2], D, dt=f32)
         self.layers = nn.ModuleList(
             [HybridLayer(spec, ls, dtype, device) for ls in spec.layers])
 
@@ -794,7 +922,8 @@ class HybridLM(nn.Module):
         entries carry an index tuple instead of a row range."""
         table = {"nedasun": _nedasun_named_slices, "kakilorn": _kakilorn_named_slices,
                  "legilix": _legilix_named_slices,
-                 "sagedra": _sagedra_named_slices}.get(self.spec.design)
+                 "sagedra": _sagedra_named_slices,
+                 "pedazen": _pedazen_named_slices}.get(self.spec.design)
         if table is not None:
             return table(self)
         out = {"embed": (self.embed, None), "embed.norm": (self.embed_norm_w, None),
@@ -838,6 +967,8 @@ class HybridLM(nn.Module):
             return param
         if where == "flat":
             return param.view(-1, param.shape[-1])
+        if isinstance(where, torch.Size):       # the parameter under another shape
+            return param.view(where)
         r0, n = where
         return param[r0:r0 + n]
 
@@ -894,6 +1025,10 @@ class HybridLM(nn.Module):
                 r = 1.0 + 0.1 * r
             elif last == "conv":
                 r *= 0.5
+            elif last == "lam":         # slow decays of a linear recurrent unit
+                r = 0.5 * r - 4.0
+            elif name.endswith(("q.norm", "k.norm")):
+                r = 1.0 + 0.1 * r
             elif dst.dim() >= 2 and "canon" not in name:
                 r *= 1.0 / math.sqrt(dst.shape[-1])
             elif (name.endswith("dkv.norm") or name.endswith("mix.norm")
@@ -1450,6 +1585,16 @@ def _heads_from_config(i, mc):
     return dict(heads=heads, kv_heads=kvh, dim=int(mc["dim"]), vdim=int(mc["vdim"]))
 
 
+def _loop_from_config(cfg) -> Optional[tuple]:
+    loop = cfg.get("loop")
+    if not loop:
+        return None
+    loop = (int(loop["start"]), int(loop["stop"]), int(loop["times"]))
+    if not (0 <= loop[0] <= loop[1] <= len(cfg["layers"])) or loop[2] < 1:
+        raise ValueError("loop: needs 0 <= start <= stop <= layers and times >= 1")
+    return loop
+
+
 def sagedra_spec_from_config(cfg: dict, name: str = "sagedra") -> HybridSpec:
     """Map a Sagedra ``config.json`` onto the generic layer specs."""
     layers = []
@@ -1491,11 +1636,7 @@ def sagedra_spec_from_config(cfg: dict, name: str = "sagedra") -> HybridSpec:
                 raise ValueError(f"layer {i}: unknown mlp kind {fc.get('kind')!r}")
             mlp = GluSpec(ff=int(fc["ff"]), act="gelu_tanh")
         layers.append(LayerSpec(mixer, mlp))
-    loop = cfg.get("loop")
-    if loop:
-        loop = (int(loop["start"]), int(loop["stop"]), int(loop["times"]))
-        if not (0 <= loop[0] <= loop[1] <= len(layers)) or loop[2] < 1:
-            raise ValueError("loop: needs 0 <= start <= stop <= layers and times >= 1")
+    loop = _loop_from_config(cfg)
     streams = int(cfg.get("streams") or 1)
     if not 1 <= streams <= MAX_STREAMS:
         raise ValueError(f"streams must be in [1, {MAX_STREAMS}]")
@@ -1505,7 +1646,7 @@ def sagedra_spec_from_config(cfg: dict, name: str = "sagedra") -> HybridSpec:
                       conv_taps=0, layers=tuple(layers), block="hyper",
                       design="sagedra", norm_offset=0.0, norm_center=True,
                       embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)),
-                      streams=streams, loop=loop or None,
+                      streams=streams, loop=loop,
                       logit_softcap=float(cfg.get("logit_softcap") or 0.0))
 
 
@@ -1603,3 +1744,161 @@ def load_sagedra_checkpoint(path: str, dtype=torch.bfloat16, device=None) -> Hyb
 
 def save_sagedra_checkpoint(model: HybridLM, path: str) -> None:
     _save_design(model, path, sagedra_config_from_spec)
+
+
+# ---------------------------------------------------------------- Pedazen
+
+def pedazen_spec_from_config(cfg: dict, name: str = "pedazen") -> HybridSpec:
+    """Map a Pedazen ``config.json`` onto the generic layer specs."""
+    layers = []
+    for i, lc in enumerate(cfg["layers"]):
+        mc, typ = lc["mixer"], lc["type"]
+        if typ == "lightning":
+            mixer = LinearAttentionSpec(
+                heads=int(mc["heads"]), dim=int(mc["dim"]), vdim=int(mc["vdim"]),
+                decay=tuple(float(v) for v in mc["decay"]))
+            if len(mixer.decay) != mixer.heads:
+                raise ValueError(f"layer {i}: decay needs one factor per head")
+        elif typ == "parallel":
+            lm, rm = mc["left"], mc["right"]
+            rot = lm.get("rot") or {}
+            left = WindowAttentionSpec(
+                **_heads_from_config(i, lm), scale=float(lm["scale"]), qk_norm=True,
+                rope_dims=int(rot.get("dims") or 0),
+                rope_base=float(rot.get("base") or 10000.0),
+                chunk=int((lm.get("mask") or {}).get("size") or 0),
+                softcap=float(lm.get("softcap") or 0.0), sink=True)
+            if left.rope_dims > left.dim or left.rope_dims % 2:
+                raise ValueError(f"layer {i}: rot.dims must be even and <= dim")
+            right = LinearUnitSpec(width=int(rm["width"]), blocks=int(rm["blocks"]),
+                                   taps=int(rm["conv"]))
+            if right.blocks < 1 or right.width % right.blocks:
+                raise ValueError(f"layer {i}: blocks must divide the unit's width")
+            if right.taps < 1:
+                raise ValueError(f"layer {i}: conv needs at least one tap")
+            mixer = ParallelMixerSpec(left, right, 0.5, 0.5, out_norm=True)
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {typ!r}")
+        fc, mlp = lc.get("mlp"), None
+        if fc is not None and fc.get("kind") == "dense":
+            mlp = GluSpec(ff=int(fc["ff"]), act="gelu_tanh")
+        elif fc is not None and fc.get("kind") == "moe":
+            rc = fc["router"]
+            gc = rc.get("groups")
+            mlp = MoESpec(experts=int(rc["experts"]), top=int(rc["top"]),
+                          ff=int(fc["expert"]["ff"]), routing="all", renorm=True,
+                          groups=(int(gc["count"]), int(gc["keep"])) if gc else None,
+                          expert="relu2")
+            if not 1 <= mlp.top <= mlp.experts:
+                raise ValueError(f"layer {i}: top must be in [1, experts]")
+            if mlp.groups is not None:
+                n, keep = mlp.groups
+                if (n < 1 or mlp.experts % n or not 1 <= keep <= n
+                        or keep * (mlp.experts // n) < mlp.top):
+                    raise ValueError(f"layer {i}: groups must divide the experts and "
+                                     f"the kept ones hold at least top of them")
+        elif fc is not None:
+            raise ValueError(f"layer {i}: unknown mlp kind {fc.get('kind')!r}")
+        layers.append(LayerSpec(mixer, mlp))
+    return HybridSpec(name=name, vocab_size=int(cfg["vocab"]),
+                      width=int(cfg["width"]),
+                      norm_eps=float(cfg["norm"]["eps"]), residual_mult=1.0,
+                      conv_taps=0, layers=tuple(layers), block="parallel",
+                      design="pedazen",
+                      embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)),
+                      tied_head=True, loop=_loop_from_config(cfg), loop_inject=True)
+
+
+def pedazen_config_from_spec(spec: HybridSpec) -> dict:
+    """Inverse of :func:`pedazen_spec_from_config` (checkpoint saving)."""
+    layers = []
+    for ls in spec.layers:
+        m = ls.mixer
+        if isinstance(m, ParallelMixerSpec):
+            a, r = m.left, m.right
+            left = {"heads": a.heads, "kv_heads": a.kv_heads, "dim": a.dim,
+                    "vdim": a.vdim, "scale": a.scale,
+                    "rot": {"base": a.rope_base, "dims": a.rope_dims}}
+            if a.chunk:
+                left["mask"] = {"size": a.chunk}
+            if a.softcap:
+                left["softcap"] = a.softcap
+            mc = {"left": left, "right": {"width": r.width, "blocks": r.blocks,
+                                          "conv": r.taps}}
+            typ = "parallel"
+        else:
+            mc = {"heads": m.heads, "dim": m.dim, "vdim": m.vdim,
+                  "decay": list(m.decay)}
+            typ = "lightning"
+        f, fc = ls.mlp, None
+        if isinstance(f, GluSpec):
+            fc = {"kind": "dense", "ff": f.ff}
+        elif f is not None:
+            rc = {"experts": f.experts, "top": f.top}
+            if f.groups is not None:
+                rc["groups"] = {"count": f.groups[0], "keep": f.groups[1]}
+            fc = {"kind": "moe", "expert": {"ff": f.ff}, "router": rc}
+        layers.append({"type": typ, "mixer": mc, "mlp": fc})
+    out = {"architecture": "Pedazen", "embedding": {"scale": spec.embed_scale},
+           "layers": layers, "norm": {"eps": spec.norm_eps},
+           "vocab": spec.vocab_size, "width": spec.width}
+    if spec.loop:
+        out["loop"] = dict(zip(("start", "stop", "times"), spec.loop))
+    return out
+
+
+def _pedazen_named_slices(model: "HybridLM") -> Dict[str, tuple]:
+    out = {"embed": (model.embed, None), "final.norm": (model.final_norm_w, None)}
+    if model.spec.loop is not None:
+        out["loop.step"] = (model.loop_step, None)
+
+    def rows(x, mat, r0, parts):
+        for nm, n in parts:
+            out[x + nm] = (mat, (r0, n))
+            r0 += n
+
+    for i, (ls, L) in enumerate(zip(model.spec.layers, model.layers)):
+        p, m = f"l{i}.", ls.mixer
+        x = p + "mix."
+        out[p + "norm1"] = (L.norm_w, None)
+        if isinstance(m, ParallelMixerSpec):
+            a, u, W = m.left, m.right, L.right
+            rows(x + "left.", L.in_w, 0, (("q", a.q_size), ("k", a.k_size),
+                                          ("v", a.v_size)))
+            y = x + "left."
+            out[y + "q.norm"] = (L.left.q_norm_w, None)
+            out[y + "k.norm"] = (L.left.k_norm_w, None)
+            out[y + "sink"], out[y + "o"] = (L.left.sink, None), (L.left.out_w, None)
+            out[y + "out"] = (L.left_norm_w, None)
+            y, n = x + "right.", u.block_size
+            rows(y, L.in_w, a.in_size, (("y", u.width), ("x", u.width)))
+            # the attention side's rows of the packed bias stay zero
+            rows(y, L.in_b, a.in_size, (("y.b", u.width), ("x.b", u.width)))
+            out[y + "conv"], out[y + "conv.b"] = (W.conv_w, None), (W.conv_b, None)
+            for k, nm in enumerate(("ra", "ri")):
+                out[y + nm] = (W.gates_w[k], None)
+                out[y + nm + ".b"] = (W.gates_b[k], torch.Size((u.blocks, n)))
+            out[y + "lam"], out[y + "o"] = (W.lam, None), (W.out_w, None)
+            out[y + "out"] = (L.right_norm_w, None)
+        else:
+            rows(x, L.in_w, 0, (("q", m.q_size), ("k", m.q_size), ("v", m.v_size),
+                                ("g", m.v_size)))
+            out[x + "norm"], out[x + "o"] = (L.onorm_w, None), (L.out_w, None)
+        f, x = ls.mlp, p + "mlp."
+        if isinstance(f, GluSpec):
+            rows(x, L.gu_w, 0, (("gate", f.ff), ("up", f.ff)))
+            out[x + "down"] = (L.down_w, None)
+        elif f is not None:
+            out[x + "router"] = (L.router_w, None)
+            for e in range(f.experts):
+                out[f"{x}e{e}.up"] = (L.exp_gu[e], None)
+                out[f"{x}e{e}.down"] = (L.exp_down[e], None)
+    return out
+
+
+def load_pedazen_checkpoint(path: str, dtype=torch.bfloat16, device=None) -> HybridLM:
+    return _load_design(path, "pedazen", pedazen_spec_from_config, dtype, device)
+
+
+def save_pedazen_checkpoint(model: HybridLM, path: str) -> None:
+    _save_design(model, path, pedazen_config_from_spec)

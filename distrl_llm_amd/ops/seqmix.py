@@ -287,11 +287,15 @@ def sigmoid_attention(q, cache, heads, kv_heads, dim, vdim, block_tables,
                                window, keep_first, slopes, pos_bias, out_dtype)
 
 
-def moe_route_all(h, router_w, correction, top, scale):
+def moe_route_all(h, router_w, correction, top, scale, groups=None, renorm=False):
+    """``groups`` = (count, keep): only outputs of the ``keep`` best of
+    ``count`` groups of neighbours are chosen; ``renorm``: the chosen scores
+    are divided by their sum."""
     if h.is_cuda:
+        n, keep = groups if groups is not None else (1, 1)
         return _ext("moe_route_all").moe_route_all(h, router_w, correction,
-                                                   top, scale)
-    return R.moe_route_all(h, router_w, correction, top, scale)
+                                                   top, scale, n, keep, renorm)
+    return R.moe_route_all(h, router_w, correction, top, scale, groups, renorm)
 
 
 def moe_experts_glu(h, idx, wts, exp_gu, exp_down, limit):
@@ -330,23 +334,27 @@ def qk_prepare_kv_write(proj, heads, kv_heads, dim, vdim, q_norm_w, k_norm_w,
 def window_attention(q, cache, heads, kv_heads, dim, vdim, whole_key,
                      block_tables, block_size, cu, tok_seq, positions, scale,
                      window, keep_first, r1, r2, gate, out_dtype, tiles=None,
-                     max_tile=0, maps=1, lam_w=None, diff=0.0, eps=0.0):
+                     max_tile=0, maps=1, lam_w=None, diff=0.0, eps=0.0,
+                     chunk=0, softcap=0.0, sink=None):
     """``tiles`` (from :func:`query_tiles` with ``WIDE_QUERY_TILE``) selects
     the tiled MFMA kernel for bf16 prompt portions; steps of few tokens per
     row run one workgroup per (token, kv head, share of the keys), fp32
     models and odd sizes one wave per (token, head). ``gate`` ([T, H] or one
     per entry, [T, H vdim]) may be a column slice of a wider matrix. ``maps``
     = 2 (with ``lam_w`` fp32 [4, dim], ``diff`` and ``eps``): differential
-    attention, two query/key maps per head over the same values."""
+    attention, two query/key maps per head over the same values. ``chunk`` >
+    0: a query sees its own chunk of positions only; ``softcap`` > 0: scores
+    become softcap tanh(score / softcap); ``sink`` (fp32 [H]) joins the
+    softmax denominator."""
     if q.is_cuda:
         return _ext("window_attention").window_attention(
             q, cache, heads, kv_heads, dim, vdim, whole_key, block_tables,
             block_size, tok_seq, positions, scale, window, keep_first, r1, r2,
-            gate, tiles, max_tile, maps, lam_w, diff, eps)
+            gate, tiles, max_tile, maps, lam_w, diff, eps, chunk, softcap, sink)
     return R.window_attention(q, cache, heads, kv_heads, dim, vdim, whole_key,
                               block_tables, block_size, cu, positions, scale,
                               window, keep_first, r1, r2, gate, out_dtype,
-                              maps, lam_w, diff, eps)
+                              maps, lam_w, diff, eps, chunk, softcap, sink)
 
 
 def gelu_tanh(x):
@@ -422,3 +430,77 @@ def hyper_close_norm(x, rows, norm_w, eps, out_dtype, center):
         return _ext("hyper_close_norm").hyper_close_norm(
             x, rows, norm_w, eps, _bf16(out_dtype), center)
     return R.hyper_close_norm(x, rows, norm_w, eps, out_dtype, center)
+
+
+# ------------------------------------------- parallel block, linear mixers
+
+def parallel_start(embed, tokens, scale, step, norm_w, eps, out_dtype, offset=1.0):
+    """Scaled embedding rows (+ the fp32 vector ``step``) as the fp32
+    residual, and their offset RMS norm in ``out_dtype``."""
+    if embed.is_cuda:
+        return _ext("parallel_start").parallel_start(
+            embed, tokens, scale, step, norm_w, eps, _bf16(out_dtype), offset)
+    return R.parallel_start(embed, tokens, scale, step, norm_w, eps, out_dtype,
+                            offset)
+
+
+def parallel_residual_norm(x, y, y2, y_w, y2_w, y_scale, y2_scale, f, inject,
+                           next_w, eps, out_dtype, offset=1.0):
+    """Fused layer tail of the parallel block (in place on the fp32 residual
+    x): x += y_scale y (+ y2_scale y2) (+ f), y and y2 RMS-normed over the
+    width first where they have a weight; ``inject`` = (embed or None,
+    tokens, scale, step) then adds scale * embed[token] and the fp32 vector
+    step; with ``next_w`` the next layer's offset RMS norm is returned."""
+    if x.is_cuda:
+        embed, tokens, scale, step = inject if inject is not None else (None, None, 1.0, None)
+        return _ext("parallel_residual_norm").parallel_residual_norm(
+            x, y, y2, y_w, y2_w, y_scale, y2_scale, f, embed, tokens, scale,
+            step, next_w, eps, _bf16(out_dtype), offset)
+    return R.parallel_residual_norm(x, y, y2, y_w, y2_w, y_scale, y2_scale, f,
+                                    inject, next_w, eps, out_dtype, offset)
+
+
+LINEAR_CHUNK = 64  # tokens the chunked linear attention kernel takes at once
+
+
+def decay_powers(decay, device):
+    """fp32 [H, LINEAR_CHUNK + 1]: powers 0 .. LINEAR_CHUNK of every head's
+    decay, formed in double precision."""
+    d = torch.tensor(decay, dtype=torch.float64)[:, None]
+    n = torch.arange(LINEAR_CHUNK + 1, dtype=torch.float64)[None]
+    return torch.pow(d, n).to(torch.float32).to(device)
+
+
+def linear_attention(proj, heads, dim, vdim, powers, norm_w, eps, state, cu,
+                     slots, out_dtype, max_tile=0):
+    """``proj`` rows [q | k | v | gate] may be a column slice of a wider
+    matrix; ``powers`` from :func:`decay_powers`. ``max_tile`` (largest tile
+    of the step's rows): bf16 steps with more than a few tokens per row run
+    the chunked MFMA kernel, others walk the tokens one by one."""
+    if proj.is_cuda:
+        return _ext("linear_attention").linear_attention(
+            proj, heads, dim, vdim, powers, norm_w, eps, state, cu, slots, max_tile)
+    return R.linear_attention(proj, heads, dim, vdim, powers, norm_w, eps, state,
+                              cu, slots, out_dtype)
+
+
+def linear_unit(proj, conv_w, conv_b, tails, gates_w, gates_b, lam, c, state, cu,
+                tok_seq, slots, out_dtype, tiles=None, tile_cu=None):
+    """``proj`` rows [y | x] may be a column slice of a wider matrix. Every
+    row of the step holds at least one token. ``tiles`` / ``tile_cu`` (from
+    :func:`query_tiles` with ``WIDE_QUERY_TILE``, and each row's first tile):
+    bf16 prompt steps form gates and prefix products per tile on MFMA."""
+    if proj.is_cuda:
+        return _ext("linear_unit").linear_unit(
+            proj, conv_w, conv_b, tails, gates_w, gates_b, lam, c, state, cu,
+            tok_seq, slots, tiles, tile_cu)
+    return R.linear_unit(proj, conv_w, conv_b, tails, gates_w, gates_b, lam, c,
+                         state, cu, slots, out_dtype)
+
+
+def moe_experts_relu2(h, idx, wts, exp_up, exp_down):
+    """Mixture of two-matrix experts down(relu(up h)^2)."""
+    if h.is_cuda:
+        return _ext("moe_experts_relu2").moe_experts_relu2(h, idx, wts, exp_up,
+                                                           exp_down)
+    return R.moe_experts_relu2(h, idx, wts, exp_up, exp_down)

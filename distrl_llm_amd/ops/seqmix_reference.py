@@ -463,15 +463,28 @@ def sigmoid_attention(q, cache, heads, kv_heads, dim, vdim, block_tables,
     return out.reshape(T, heads * vdim).to(out_dtype)
 
 
-def moe_route_all(h, router_w, correction, top, scale):
+def moe_route_all(h, router_w, correction, top, scale, groups=None, renorm=False):
     """fp32 router over every output: s = softmax(W h); the ``top`` largest
     s + correction are chosen (ties: lowest index first); weights =
-    s[chosen] * scale, not renormalised."""
+    s[chosen] * scale, with ``renorm`` divided by their sum (+ 1e-20) first.
+    ``groups`` = (count, keep): outputs form ``count`` equal groups of
+    neighbours, only those of the ``keep`` groups with the largest single
+    corrected score can be chosen."""
     s = torch.softmax(F.linear(h.float(), router_w.float()), -1)
     c = s if correction is None else s + correction.float()
+    if groups is not None:
+        n, keep = groups
+        best = c.view(c.shape[0], n, -1).amax(-1)
+        _, order = torch.sort(best, dim=-1, descending=True, stable=True)
+        ok = torch.zeros_like(best, dtype=torch.bool)
+        ok.scatter_(1, order[:, :keep], True)
+        c = c.masked_fill(~ok.repeat_interleave(c.shape[1] // n, 1), float("-inf"))
     _, idx = torch.sort(c, dim=-1, descending=True, stable=True)
     idx = idx[:, :top]
-    return idx.to(torch.int32), torch.gather(s, 1, idx) * scale
+    wts = torch.gather(s, 1, idx)
+    if renorm:
+        wts = wts / (wts.sum(-1, keepdim=True) + 1e-20)
+    return idx.to(torch.int32), wts * scale
 
 
 def moe_experts_glu(h, idx, wts, exp_gu, exp_down, limit):
@@ -566,11 +579,14 @@ def qk_prepare_kv_write(proj, heads, kv_heads, dim, vdim, q_norm_w, k_norm_w,
 def window_attention(q, cache, heads, kv_heads, dim, vdim, whole_key,
                      block_tables, block_size, cu, positions, scale, window,
                      keep_first, r1, r2, gate, out_dtype, maps=1, lam_w=None,
-                     diff=0.0, eps=0.0):
+                     diff=0.0, eps=0.0, chunk=0, softcap=0.0, sink=None):
     """Grouped-query softmax attention over paged [k | v] rows.
 
     Query i sees the keys j <= i with i - j < window or j < keep_first
-    (window 0: all j <= i). score = q . k * scale, where head h meets the
+    (window 0: all j <= i); ``chunk`` > 0: those of its own chunk,
+    floor(j / chunk) = floor(i / chunk), or j < keep_first. ``softcap`` > 0:
+    scaled scores become softcap * tanh(score / softcap); ``sink`` (fp32 [H])
+    adds exp(sink[h]) to the softmax denominator. score = q . k * scale, where head h meets the
     keys of its own kv head, or with ``whole_key`` (q rows of kv_heads * dim
     entries) the whole key row; ``r1``/``r2`` (fp32 [H]) take
     r1 ln(1 + r2 (i - j)) off the score; ``gate`` ([T, H] or, one per entry,
@@ -596,7 +612,8 @@ def window_attention(q, cache, heads, kv_heads, dim, vdim, whole_key,
             a.append(window_attention(
                 q.view(T, heads, 2, dim)[:, :, m], one, heads, kv_heads, dim, vdim,
                 False, block_tables, block_size, cu, positions, scale, window,
-                keep_first, None, None, None, torch.float32).view(T, heads, vdim))
+                keep_first, None, None, None, torch.float32, chunk=chunk,
+                softcap=softcap, sink=sink).view(T, heads, vdim))
         out = a[0] - lam * a[1]
         out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps) * (1.0 - diff)
         if gate is not None:
@@ -619,6 +636,8 @@ def window_attention(q, cache, heads, kv_heads, dim, vdim, whole_key,
             k = kv[:, :nk].view(-1, kv_heads, dim).repeat_interleave(rep, 1)
             s = torch.einsum("thd,jhd->htj", q[a:e].float(), k) * scale
         p = positions[a:e].long()[:, None]
+        if softcap > 0:
+            s = softcap * torch.tanh(s / softcap)
         if r1 is not None:
             dist = (p - j[None, :]).clamp(min=0).float()
             s = s - r1.float()[:, None, None] * torch.log1p(
@@ -626,8 +645,12 @@ def window_attention(q, cache, heads, kv_heads, dim, vdim, whole_key,
         ok = j[None, :] <= p
         if window > 0:
             ok = ok & ((p - j[None, :] < window) | (j[None, :] < keep_first))
+        if chunk > 0:
+            ok = ok & ((j[None, :] >= p // chunk * chunk) | (j[None, :] < keep_first))
         s = s.masked_fill(~ok[None], float("-inf"))
-        out[a:e] = torch.einsum("htj,jhd->thd", torch.softmax(s, -1), v)
+        if sink is not None:
+            s = torch.cat([s, sink.float()[:, None, None].expand(-1, e - a, 1)], -1)
+        out[a:e] = torch.einsum("htj,jhd->thd", torch.softmax(s, -1)[..., :j.numel()], v)
     if gate is not None:
         out = out * torch.sigmoid(gate.float().reshape(T, heads, -1))
     return out.reshape(T, heads * vdim).to(out_dtype)
@@ -729,3 +752,115 @@ def hyper_residual_norm(x, y, y2, y_w, y2_w, y_scale, y2_scale, mix, out_w,
 def hyper_close_norm(x, rows, norm_w, eps, out_dtype, center):
     """norm(sum of the streams) of the given rows."""
     return row_norm(x[rows].sum(1), norm_w, eps, center).to(out_dtype)
+
+
+# ------------------------------------------------- parallel block, linear mixers
+
+def parallel_start(embed, tokens, scale, step, norm_w, eps, out_dtype, offset=1.0):
+    """(x = scale * embed[token] (+ step) in fp32, x / rms(x) * (offset +
+    norm_w) in ``out_dtype``)."""
+    x = embed[tokens].float() * scale
+    if step is not None:
+        x = x + step.float()
+    return x, offset_rmsnorm(x, norm_w, eps, out_dtype, offset)[1]
+
+
+def parallel_residual_norm(x, y, y2, y_w, y2_w, y_scale, y2_scale, f, inject,
+                           next_w, eps, out_dtype, offset=1.0):
+    """Layer tail of the parallel block on the fp32 residual, in place:
+    x += y_scale y (+ y2_scale y2) (+ f), y and y2 RMS-normed over the width
+    first where a weight (``y_w``/``y2_w``) is given; then ``inject`` =
+    (embed, tokens, scale, step): x += scale * embed[token] + step (``embed``
+    None: only the step). With ``next_w`` returns x / rms(x) * (offset +
+    next_w) in ``out_dtype``, else None."""
+    def side(v, w, a):
+        v = v.float()
+        if w is not None:
+            v = v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+        return a * v
+
+    if y is not None:
+        x.add_(side(y, y_w, y_scale))
+    if y2 is not None:
+        x.add_(side(y2, y2_w, y2_scale))
+    if f is not None:
+        x.add_(f.float())
+    if inject is not None:
+        embed, tokens, scale, step = inject
+        if embed is not None:
+            x.add_(embed[tokens].float() * scale)
+        x.add_(step.float())
+    if next_w is None:
+        return None
+    return offset_rmsnorm(x, next_w, eps, out_dtype, offset)[1]
+
+
+def linear_attention(proj, heads, dim, vdim, powers, norm_w, eps, state, cu,
+                     slots, out_dtype):
+    """Linear attention with a fixed decay per head over packed projection
+    rows [q | k | v | gate]: q, k, v = silu; per head S <- decay S + k v^T,
+    o = S^T q; the heads' outputs are RMS-normed together (plain ``norm_w``
+    [H vdim]) and scaled by sigmoid(gate). ``powers`` fp32 [H, n]: powers
+    0, 1, ... of the decay; state fp32 [slots, H * vdim * dim] (per head
+    value-major: S^T), advanced in place. -> [T, H * vdim]."""
+    T = proj.shape[0]
+    nq, nv = heads * dim, heads * vdim
+    x = proj[:, :2 * nq + nv].float()
+    x = x * torch.sigmoid(x)
+    q, k = x[:, :nq].view(T, heads, dim), x[:, nq:2 * nq].view(T, heads, dim)
+    v = x[:, 2 * nq:].view(T, heads, vdim)
+    decay = powers[:, 1].float()[:, None, None]
+    o = torch.empty(T, heads, vdim, dtype=torch.float32, device=proj.device)
+    cu_l, slots_l = cu.tolist(), slots.tolist()
+    for b, s in enumerate(slots_l):
+        S = state[s].view(heads, vdim, dim).clone()
+        for t in range(cu_l[b], cu_l[b + 1]):
+            S = decay * S + v[t][:, :, None] * k[t][:, None, :]
+            o[t] = torch.einsum("hvk,hk->hv", S, q[t])
+        state[s] = S.reshape(-1)
+    o = o.view(T, nv)
+    o = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * norm_w.float()
+    return (o * torch.sigmoid(proj[:, 2 * nq + nv:2 * nq + 2 * nv].float())).to(out_dtype)
+
+
+def linear_unit(proj, conv_w, conv_b, tails, gates_w, gates_b, lam, c, state, cu,
+                slots, out_dtype):
+    """Real-gated linear recurrent unit over projection rows [y | x] (biases
+    added): u = conv(x) + conv_b (causal, ``tails`` advanced), r and i =
+    sigmoids of the block-diagonal maps ``gates_w`` [2, blocks, n, n] of u
+    plus ``gates_b`` [2, width]; log a = -c r softplus(lam);
+    S <- a S + sqrt(1 - a^2) i u (``state`` fp32 [slots, width], advanced in
+    place); result S * gelu_tanh(y)."""
+    T = proj.shape[0]
+    W = conv_w.shape[0]
+    n = gates_w.shape[-1]
+    u = tap_conv(proj[:, W:2 * W], conv_w, tails, cu, slots) + conv_b.float()
+    g = torch.einsum("tbk,gbnk->gtbn", u.view(T, -1, n), gates_w.float())
+    g = torch.sigmoid(g.reshape(2, T, W) + gates_b.float()[:, None])
+    log_a = -c * g[0] * F.softplus(lam.float())
+    a = torch.exp(log_a)
+    b = torch.sqrt(-torch.expm1(2.0 * log_a)) * g[1] * u
+    out = torch.empty(T, W, dtype=torch.float32, device=proj.device)
+    cu_l, slots_l = cu.tolist(), slots.tolist()
+    for r, s in enumerate(slots_l):
+        S = state[s]
+        for t in range(cu_l[r], cu_l[r + 1]):
+            S = a[t] * S + b[t]
+            out[t] = S
+        state[s] = S
+    return (out * gelu_tanh(proj[:, :W].float())).to(out_dtype)
+
+
+def moe_experts_relu2(h, idx, wts, exp_up, exp_down):
+    """sum_k wts[t, k] * down_e(relu(up_e h)^2), e = idx[t, k]. exp_up
+    [E, ff, D], exp_down [E, D, ff]. Returns fp32 [T, D]."""
+    out = torch.zeros(h.shape, dtype=torch.float32, device=h.device)
+    for e in range(exp_up.shape[0]):
+        hit = idx == e
+        rows = hit.any(-1).nonzero().flatten()
+        if rows.numel() == 0:
+            continue
+        a = torch.relu(F.linear(h[rows], exp_up[e]).float())
+        y = F.linear((a * a).to(h.dtype), exp_down[e]).float()
+        out[rows] += (wts[rows] * hit[rows]).sum(-1, keepdim=True) * y
+    return out

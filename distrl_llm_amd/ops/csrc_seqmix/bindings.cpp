@@ -42,7 +42,10 @@ torch::Tensor moe_experts(torch::Tensor h, torch::Tensor idx, torch::Tensor wts,
 
 std::vector<torch::Tensor> moe_route_all(torch::Tensor h, torch::Tensor router_w,
                                          c10::optional<torch::Tensor> correction,
-                                         int64_t top, double scale);
+                                         int64_t top, double scale, int64_t groups,
+                                         int64_t keep_groups, bool renorm);
+torch::Tensor moe_experts_relu2(torch::Tensor h, torch::Tensor idx, torch::Tensor wts,
+                                torch::Tensor exp_up, torch::Tensor exp_down);
 torch::Tensor moe_experts_glu(torch::Tensor h, torch::Tensor idx, torch::Tensor wts,
                               torch::Tensor exp_gu, torch::Tensor exp_down, double limit);
 torch::Tensor tap_conv_silu(torch::Tensor x, torch::Tensor w, torch::Tensor tails,
@@ -78,7 +81,26 @@ torch::Tensor window_attention(torch::Tensor q, torch::Tensor cache, int64_t hea
                                c10::optional<torch::Tensor> gate,
                                c10::optional<torch::Tensor> tiles, int64_t max_tile_queries,
                                int64_t maps, c10::optional<torch::Tensor> lam_w, double diff,
-                               double eps);
+                               double eps, int64_t chunk, double softcap,
+                               c10::optional<torch::Tensor> sink);
+std::vector<torch::Tensor> parallel_start(torch::Tensor embed, torch::Tensor tokens, double scale,
+                                          c10::optional<torch::Tensor> step, torch::Tensor norm_w,
+                                          double eps, bool out_bf16, double offset);
+c10::optional<torch::Tensor> parallel_residual_norm(
+    torch::Tensor x, c10::optional<torch::Tensor> y, c10::optional<torch::Tensor> y2,
+    c10::optional<torch::Tensor> y_w, c10::optional<torch::Tensor> y2_w, double y_scale,
+    double y2_scale, c10::optional<torch::Tensor> f, c10::optional<torch::Tensor> embed,
+    c10::optional<torch::Tensor> tokens, double scale, c10::optional<torch::Tensor> step,
+    c10::optional<torch::Tensor> norm_w, double eps, bool out_bf16, double offset);
+torch::Tensor linear_attention(torch::Tensor proj, int64_t heads, int64_t dim, int64_t vdim,
+                               torch::Tensor powers, torch::Tensor norm_w, double eps,
+                               torch::Tensor state, torch::Tensor cu, torch::Tensor slots,
+                               int64_t max_tile);
+torch::Tensor linear_unit(torch::Tensor proj, torch::Tensor conv_w, torch::Tensor conv_b,
+                          torch::Tensor tails, torch::Tensor gates_w, torch::Tensor gates_b,
+                          torch::Tensor lam, double c, torch::Tensor state, torch::Tensor cu,
+                          torch::Tensor tok_seq, torch::Tensor slots,
+                          c10::optional<torch::Tensor> tiles, c10::optional<torch::Tensor> tile_cu);
 torch::Tensor gelu_glu(torch::Tensor gu);
 torch::Tensor cap_logits(torch::Tensor z, double scale, double cap);
 std::vector<torch::Tensor> hyper_start(torch::Tensor embed, torch::Tensor tokens, double scale,
@@ -163,6 +185,13 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("hyper_residual_norm", &hyper_residual_norm,
         "stream update of a sublayer's output + next read sum and norm");
   m.def("hyper_close_norm", &hyper_close_norm, "norm of the streams' sum");
+  m.def("moe_experts_relu2", &moe_experts_relu2, "grouped-GEMM mixture of squared-ReLU experts");
+  m.def("parallel_start", &parallel_start, "scaled embedding rows + first norm");
+  m.def("parallel_residual_norm", &parallel_residual_norm,
+        "parallel block's layer tail: normed sides, feed-forward, pass injection, next norm");
+  m.def("linear_attention", &linear_attention,
+        "linear attention with fixed decays, fp32 state per slot, gated RMS norm");
+  m.def("linear_unit", &linear_unit, "real-gated linear recurrent unit with short convolution");
   m.def("window_attention", &window_attention,
-        "paged GQA softmax attention: window with kept first tokens, log distance bias, two maps, output gate");
+        "paged GQA softmax attention: window or chunks, kept first tokens, log distance bias, cap, sink, two maps, output gate");
 }

@@ -18,44 +18,6 @@
 
 namespace {
 
-template <int VEC> struct hs_f { float v[VEC]; };
-
-template <int VEC> SM_INLINE hs_f<VEC> hs_load(const float* p) {
-  hs_f<VEC> r;
-  if constexpr (VEC == 4) {
-    const float4 a = *reinterpret_cast<const float4*>(p);
-    r.v[0] = a.x; r.v[1] = a.y; r.v[2] = a.z; r.v[3] = a.w;
-  } else {
-    r.v[0] = *p;
-  }
-  return r;
-}
-template <int VEC> SM_INLINE hs_f<VEC> hs_load(const bf16_t* p) {
-  hs_f<VEC> r;
-  if constexpr (VEC == 4) {
-    const uint2 a = *reinterpret_cast<const uint2*>(p);
-    r.v[0] = __uint_as_float(a.x << 16); r.v[1] = __uint_as_float(a.x & 0xffff0000u);
-    r.v[2] = __uint_as_float(a.y << 16); r.v[3] = __uint_as_float(a.y & 0xffff0000u);
-  } else {
-    r.v[0] = to_f(*p);
-  }
-  return r;
-}
-template <int VEC> SM_INLINE void hs_store(float* p, const hs_f<VEC>& r) {
-  if constexpr (VEC == 4) *reinterpret_cast<float4*>(p) = make_float4(r.v[0], r.v[1], r.v[2], r.v[3]);
-  else *p = r.v[0];
-}
-template <int VEC> SM_INLINE void hs_store(bf16_t* p, const hs_f<VEC>& r) {
-  if constexpr (VEC == 4) {
-    unsigned int w[4];
-    #pragma unroll
-    for (int k = 0; k < 4; ++k) w[k] = __bfloat16_as_ushort(__float2bfloat16(r.v[k]));
-    *reinterpret_cast<uint2*>(p) = make_uint2(w[0] | (w[1] << 16), w[2] | (w[3] << 16));
-  } else {
-    *p = __float2bfloat16(r.v[0]);
-  }
-}
-
 // h = norm(u) * w for the row u in LDS; every thread handles the entries it
 // wrote itself (same stride), sum is its share of the row's sum.
 template <typename T, int VEC>
@@ -64,17 +26,17 @@ SM_INLINE void hs_norm_out(const float* u, float sum, const float* __restrict__ 
   const float mean = center ? sm_block_sum(sum, red) / (float)D : 0.f;
   float ss = 0.f;
   for (int d = threadIdx.x * VEC; d < D; d += blockDim.x * VEC) {
-    const hs_f<VEC> v = hs_load<VEC>(u + d);
+    const sm_vec<VEC> v = sm_load<VEC>(u + d);
     #pragma unroll
     for (int k = 0; k < VEC; ++k) ss += (v.v[k] - mean) * (v.v[k] - mean);
   }
   const float inv = 1.0f / sqrtf(sm_block_sum(ss, red) / (float)D + eps);
   for (int d = threadIdx.x * VEC; d < D; d += blockDim.x * VEC) {
-    hs_f<VEC> v = hs_load<VEC>(u + d);
-    const hs_f<VEC> wv = hs_load<VEC>(w + d);
+    sm_vec<VEC> v = sm_load<VEC>(u + d);
+    const sm_vec<VEC> wv = sm_load<VEC>(w + d);
     #pragma unroll
     for (int k = 0; k < VEC; ++k) v.v[k] = (v.v[k] - mean) * inv * wv.v[k];
-    hs_store<VEC>(h + d, v);
+    sm_store<VEC>(h + d, v);
   }
 }
 
@@ -89,18 +51,18 @@ __global__ __launch_bounds__(256) void hyper_start_kernel(
   const T* e = embed + tokens[t] * D;
   float sum = 0.f;
   for (int d = threadIdx.x * VEC; d < D; d += blockDim.x * VEC) {
-    hs_f<VEC> v = hs_load<VEC>(e + d), u;
+    sm_vec<VEC> v = sm_load<VEC>(e + d), u;
     #pragma unroll
     for (int k = 0; k < VEC; ++k) { v.v[k] *= scale; u.v[k] = 0.f; }
     for (int s = 0; s < S; ++s) {
-      hs_store<VEC>(x + (t * S + s) * D + d, v);
+      sm_store<VEC>(x + (t * S + s) * D + d, v);
       const float r = read_w[s];
       #pragma unroll
       for (int k = 0; k < VEC; ++k) u.v[k] = fmaf(r, v.v[k], u.v[k]);
     }
     #pragma unroll
     for (int k = 0; k < VEC; ++k) sum += u.v[k];
-    hs_store<VEC>(hs_u + d, u);
+    sm_store<VEC>(hs_u + d, u);
   }
   hs_norm_out<T, VEC>(hs_u, sum, norm_w, eps, center != 0, D, red, h + t * D);
 }
@@ -124,11 +86,11 @@ __global__ __launch_bounds__(256) void hyper_residual_kernel(
   if (yw != nullptr || y2w != nullptr) {
     float ss = 0.f, ss2 = 0.f;
     for (int d = threadIdx.x * VEC; d < D; d += blockDim.x * VEC) {
-      const hs_f<VEC> v = hs_load<VEC>(yr + d);
+      const sm_vec<VEC> v = sm_load<VEC>(yr + d);
       #pragma unroll
       for (int k = 0; k < VEC; ++k) ss += v.v[k] * v.v[k];
       if (y2r != nullptr) {
-        const hs_f<VEC> v2 = hs_load<VEC>(y2r + d);
+        const sm_vec<VEC> v2 = sm_load<VEC>(y2r + d);
         #pragma unroll
         for (int k = 0; k < VEC; ++k) ss2 += v2.v[k] * v2.v[k];
       }
@@ -139,35 +101,35 @@ __global__ __launch_bounds__(256) void hyper_residual_kernel(
   float* xr = x + t * S * D;
   float sum = 0.f;
   for (int d = threadIdx.x * VEC; d < D; d += blockDim.x * VEC) {
-    hs_f<VEC> xs[SMAX];
+    sm_vec<VEC> xs[SMAX];
     #pragma unroll
     for (int s = 0; s < SMAX; ++s)
-      if (s < S) xs[s] = hs_load<VEC>(xr + (int64_t)s * D + d);
-    hs_f<VEC> v = hs_load<VEC>(yr + d);
+      if (s < S) xs[s] = sm_load<VEC>(xr + (int64_t)s * D + d);
+    sm_vec<VEC> v = sm_load<VEC>(yr + d);
     if (yw != nullptr) {
-      const hs_f<VEC> w = hs_load<VEC>(yw + d);
+      const sm_vec<VEC> w = sm_load<VEC>(yw + d);
       #pragma unroll
       for (int k = 0; k < VEC; ++k) v.v[k] *= w.v[k];
     }
     #pragma unroll
     for (int k = 0; k < VEC; ++k) v.v[k] *= a;
     if (y2r != nullptr) {
-      hs_f<VEC> v2 = hs_load<VEC>(y2r + d);
+      sm_vec<VEC> v2 = sm_load<VEC>(y2r + d);
       if (y2w != nullptr) {
-        const hs_f<VEC> w = hs_load<VEC>(y2w + d);
+        const sm_vec<VEC> w = sm_load<VEC>(y2w + d);
         #pragma unroll
         for (int k = 0; k < VEC; ++k) v2.v[k] *= w.v[k];
       }
       #pragma unroll
       for (int k = 0; k < VEC; ++k) v.v[k] = fmaf(a2, v2.v[k], v.v[k]);
     }
-    hs_f<VEC> u;
+    sm_vec<VEC> u;
     #pragma unroll
     for (int k = 0; k < VEC; ++k) u.v[k] = 0.f;
     #pragma unroll
     for (int q = 0; q < SMAX; ++q) {
       if (q < S) {
-        hs_f<VEC> n;
+        sm_vec<VEC> n;
         const float o = out_w[q];
         #pragma unroll
         for (int k = 0; k < VEC; ++k) n.v[k] = o * v.v[k];
@@ -179,7 +141,7 @@ __global__ __launch_bounds__(256) void hyper_residual_kernel(
             for (int k = 0; k < VEC; ++k) n.v[k] = fmaf(m, xs[s].v[k], n.v[k]);
           }
         }
-        hs_store<VEC>(xr + (int64_t)q * D + d, n);
+        sm_store<VEC>(xr + (int64_t)q * D + d, n);
         if (norm_w != nullptr) {
           const float r = read_w[q];
           #pragma unroll
@@ -190,7 +152,7 @@ __global__ __launch_bounds__(256) void hyper_residual_kernel(
     if (norm_w != nullptr) {
       #pragma unroll
       for (int k = 0; k < VEC; ++k) sum += u.v[k];
-      hs_store<VEC>(hs_u + d, u);
+      sm_store<VEC>(hs_u + d, u);
     }
   }
   if (norm_w != nullptr)
@@ -207,15 +169,15 @@ __global__ __launch_bounds__(256) void hyper_close_kernel(
   if (row < 0 || row >= T_rows) return;            // uniform over the workgroup
   float sum = 0.f;
   for (int d = threadIdx.x * VEC; d < D; d += blockDim.x * VEC) {
-    hs_f<VEC> u = hs_load<VEC>(x + row * S * D + d);
+    sm_vec<VEC> u = sm_load<VEC>(x + row * S * D + d);
     for (int s = 1; s < S; ++s) {
-      const hs_f<VEC> v = hs_load<VEC>(x + (row * S + s) * D + d);
+      const sm_vec<VEC> v = sm_load<VEC>(x + (row * S + s) * D + d);
       #pragma unroll
       for (int k = 0; k < VEC; ++k) u.v[k] += v.v[k];
     }
     #pragma unroll
     for (int k = 0; k < VEC; ++k) sum += u.v[k];
-    hs_store<VEC>(hs_u + d, u);
+    sm_store<VEC>(hs_u + d, u);
   }
   hs_norm_out<T, VEC>(hs_u, sum, norm_w, eps, center != 0, D, red,
                       h + (int64_t)blockIdx.x * D);

@@ -210,10 +210,6 @@ __global__ __launch_bounds__(256) void sandwich_residual_kernel(
   }
 }
 
-// 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))), fp32 inside.
-SM_INLINE float gelu_tanh_f(float z) {
-  return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-}
 template <typename T>
 __global__ __launch_bounds__(256) void gelu_tanh_kernel(const T* __restrict__ x, int64_t n,
                                                         T* __restrict__ out) {

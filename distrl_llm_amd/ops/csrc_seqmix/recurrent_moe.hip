@@ -1,10 +1,10 @@
 // minGRU scan over a flat varlen batch (fp32 state per slot), the fp32
 // top-k routers (softmax over the chosen logits; softmax over every output
-// with a choice correction and scaled, unnormalised weights; or plain sigmoid
-// scores), and the
+// with a choice correction and scaled weights, on request renormalised and
+// chosen within the best groups of outputs; or plain sigmoid scores), and the
 // mixture-of-experts feed-forward as two grouped GEMMs over expert-sorted
 // rows (bf16: MFMA 16x16x32 tiles; fp32: plain FMA; SiLU-gated or clamped
-// GLU experts) followed by a fixed-order weighted combine, which also adds
+// GLU experts, or ungated squared-ReLU ones) followed by a fixed-order weighted combine, which also adds
 // the identity experts' share of the input. The routing weight multiplies an
 // expert's output (in the combine) or, for designs that scale the expert's
 // input, its gate and up products before the activation.
@@ -123,7 +123,10 @@ __global__ __launch_bounds__(256) void mingru_chunk_apply_kernel(
 // one lane picks the top-k by repeated arg-max (ties: the lowest index) and
 // takes the softmax over the chosen logits.
 // ALL: scores s = softmax over all E outputs (no bias); the top-k of
-// s + corr are chosen; weights = s[chosen] * wscale, not renormalised.
+// s + corr are chosen; weights = s[chosen] * wscale, with renorm divided by
+// their sum (+ 1e-20). gcount > 1: the outputs form gcount equal groups of
+// neighbours and only the gkeep groups with the largest single s + corr can be
+// chosen from.
 // sig (not ALL): weights = sigmoid of the chosen logits, not renormalised.
 #define SM_MAX_EXPERTS 256
 template <typename T, bool ALL>
@@ -131,9 +134,11 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
     const T* __restrict__ h, const float* __restrict__ w,
     const float* __restrict__ bias, int D, int E, int top,
     int* __restrict__ idx, float* __restrict__ wts,
-    const float* __restrict__ corr, float wscale, bool sig) {
+    const float* __restrict__ corr, float wscale, bool sig, int gcount, int gkeep,
+    bool renorm) {
   __shared__ float z[SM_MAX_EXPERTS];
   __shared__ float sc[SM_MAX_EXPERTS];
+  __shared__ float gz[ALL ? SM_MAX_EXPERTS : 1];
   const int64_t t = blockIdx.x;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   for (int e = wave; e < E; e += 4) {
@@ -163,6 +168,25 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
         sc[e] /= sum;
         z[e] = sc[e] + (corr != nullptr ? corr[e] : 0.f);
       }
+      if (gcount > 1 && gkeep < gcount) {
+        // the gcount - gkeep worst groups leave the choice (ties: the highest
+        // index leaves first)
+        const int gn = E / gcount;
+        for (int g = 0; g < gcount; ++g) {
+          float m = -INFINITY;
+          for (int e = g * gn; e < (g + 1) * gn; ++e) m = fmaxf(m, z[e]);
+          gz[g] = m;
+        }
+        for (int k = 0; k < gcount - gkeep; ++k) {
+          int worst = 0;
+          float wv = INFINITY;
+          for (int g = 0; g < gcount; ++g)
+            if (gz[g] <= wv) { wv = gz[g]; worst = g; }
+          gz[worst] = NAN;              // compares false from now on
+          for (int e = worst * gn; e < (worst + 1) * gn; ++e) z[e] = -INFINITY;
+        }
+      }
+      float wsum = 0.f;
       for (int k = 0; k < top; ++k) {
         int best = -1;
         float bv = -INFINITY;
@@ -171,7 +195,12 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
         if (best < 0) best = 0;
         idx[t * top + k] = best;
         wts[t * top + k] = sc[best] * wscale;
+        wsum += sc[best];
         z[best] = -INFINITY;
+      }
+      if (renorm) {
+        const float inv = 1.0f / (wsum + 1e-20f);
+        for (int k = 0; k < top; ++k) wts[t * top + k] *= inv;
       }
     }
     return;
@@ -244,10 +273,15 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(
 //         with rw both products are scaled by rw[i] first (W (w a) = w (W a));
 //         W[e] = [gate (N rows); up (N rows)] x K;   out bf16 [M, N]
 // MODE 1: out[i, n] = a_i . W[e][n], a_i = A[i];     out fp32 [M, N]
+// MODE 2: out[i, f] = relu(a_i . W[e][f])^2, a_i = A[src[i]];   out bf16 [M, N]
 // MFMA 16x16x32 bf16 fragments: A lane l -> row l&15, k (l>>4)*8..+7;
 // B lane l -> column l&15, same k; D lane l reg r -> row (l>>4)*4+r, col l&15.
 SM_INLINE float moe_act(float g, float u, float limit) {
   return (limit > 0.f) ? sm_capped_glu(g, u, limit) : g * sm_sigmoid(g) * u;
+}
+SM_INLINE float moe_relu2(float u) {
+  u = fmaxf(u, 0.f);
+  return u * u;
 }
 SM_INLINE bf16v8 load8(const bf16_t* p, int valid, bool vec) {
   bf16v8 v;
@@ -307,7 +341,7 @@ __global__ __launch_bounds__(64 * NWV) void moe_gemm_bf16_kernel(
       const int r = v >> 3, kc = (v & 7) * 8;
       bf16v8 val;
       if (r < rows) {
-        const int64_t arow = (MODE == 0) ? src[row0 + r] : (row0 + r);
+        const int64_t arow = (MODE != 1) ? src[row0 + r] : (row0 + r);
         val = load8(A + arow * K + k0 + kc, K - (k0 + kc), vec);
       } else {
         #pragma unroll
@@ -346,6 +380,8 @@ __global__ __launch_bounds__(64 * NWV) void moe_gemm_bf16_kernel(
           const float w = (rw != nullptr) ? rw[row0 + r] : 1.0f;
           reinterpret_cast<bf16_t*>(outp)[o] =
               __float2bfloat16(moe_act(w * acc[mt][rr], w * acc2[mt][rr], limit));
+        } else if (MODE == 2) {
+          reinterpret_cast<bf16_t*>(outp)[o] = __float2bfloat16(moe_relu2(acc[mt][rr]));
         } else {
           reinterpret_cast<float*>(outp)[o] = acc[mt][rr];
         }
@@ -385,7 +421,7 @@ __global__ __launch_bounds__(256) void moe_gemm_bf16_splitk_kernel(
   const int Nw = (MODE == 0) ? 2 * N : N;
   const bf16_t* Wg = W + ((int64_t)e * Nw + (n < N ? n : 0)) * K;
   const bf16_t* Wu = Wg + (int64_t)N * K;
-  const int64_t arow = (lrow < rows) ? ((MODE == 0) ? src[row0 + lrow] : (row0 + lrow)) : -1;
+  const int64_t arow = (lrow < rows) ? ((MODE != 1) ? src[row0 + lrow] : (row0 + lrow)) : -1;
   const bf16_t* ap = A + (arow < 0 ? 0 : arow) * K;
   f32x4 acc = {0.f, 0.f, 0.f, 0.f}, acc2 = {0.f, 0.f, 0.f, 0.f};
   #pragma unroll 4
@@ -423,7 +459,9 @@ __global__ __launch_bounds__(256) void moe_gemm_bf16_splitk_kernel(
       if (MODE == 0) {
         const float w = (rw != nullptr) ? rw[row0 + r] : 1.0f;
         reinterpret_cast<bf16_t*>(outp)[o] = __float2bfloat16(moe_act(w * g, w * u, limit));
-      } else
+      } else if (MODE == 2)
+        reinterpret_cast<bf16_t*>(outp)[o] = __float2bfloat16(moe_relu2(g));
+      else
         reinterpret_cast<float*>(outp)[o] = g;
     }
   }
@@ -443,7 +481,7 @@ __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(
   int e = 0;
   while (e + 1 < E && i >= off[e + 1]) ++e;
   const int Nw = (MODE == 0) ? 2 * N : N;
-  const float* a = A + (int64_t)((MODE == 0) ? src[i] : i) * K;
+  const float* a = A + (int64_t)((MODE != 1) ? src[i] : i) * K;
   const float* wg = W + ((int64_t)e * Nw + n) * K;
   float g = 0.f, u = 0.f;
   for (int k = 0; k < K; ++k) {
@@ -451,7 +489,7 @@ __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(
     if (MODE == 0) u = fmaf(a[k], wg[(int64_t)N * K + k], u);
   }
   if (MODE == 0 && rw != nullptr) { g *= rw[i]; u *= rw[i]; }
-  out[id] = (MODE == 0) ? moe_act(g, u, limit) : g;
+  out[id] = (MODE == 0) ? moe_act(g, u, limit) : (MODE == 2) ? moe_relu2(g) : g;
 }
 
 // out[t, d] = sum_k wts[t, k] * y[inv[t * top + k], d]   (k in order; wts
@@ -545,13 +583,15 @@ torch::Tensor mingru_scan(torch::Tensor zxg, torch::Tensor bias, torch::Tensor s
 static std::vector<torch::Tensor> moe_route_impl(
     torch::Tensor h, torch::Tensor router_w, c10::optional<torch::Tensor> router_b,
     int64_t top, bool all, c10::optional<torch::Tensor> corr, double wscale,
-    bool sig = false) {
+    bool sig = false, int64_t gcount = 1, int64_t gkeep = 1, bool renorm = false) {
   SM_CHECK_CUDA(h); SM_CHECK_CUDA(router_w); SM_CHECK_F32(router_w);
   const int64_t T = h.size(0);
   const int D = h.size(1);
   const int E = router_w.size(0);
   TORCH_CHECK(router_w.size(1) == D, "moe_route: shapes");
   TORCH_CHECK(E <= SM_MAX_EXPERTS && top >= 1 && top <= E, "moe_route: experts/top");
+  TORCH_CHECK(gcount >= 1 && E % gcount == 0 && gkeep >= 1 && gkeep <= gcount &&
+              gkeep * (E / gcount) >= top, "moe_route: groups");
   const float* bp = nullptr;
   const float* cp = nullptr;
   if (router_b.has_value()) {
@@ -573,7 +613,8 @@ static std::vector<torch::Tensor> moe_route_impl(
 #define ROUTE(TY, ALLV)                                                                    \
   moe_route_kernel<TY, ALLV><<<T, 256, 0, stream>>>(                                       \
       reinterpret_cast<const TY*>(h.data_ptr()), router_w.data_ptr<float>(), bp, D, E,     \
-      (int)top, idx.data_ptr<int>(), wts.data_ptr<float>(), cp, (float)wscale, sig)
+      (int)top, idx.data_ptr<int>(), wts.data_ptr<float>(), cp, (float)wscale, sig,  \
+      (int)gcount, (int)gkeep, renorm)
   if (bf16) { if (all) ROUTE(bf16_t, true); else ROUTE(bf16_t, false); }
   else { if (all) ROUTE(float, true); else ROUTE(float, false); }
 #undef ROUTE
@@ -588,8 +629,10 @@ std::vector<torch::Tensor> moe_route(torch::Tensor h, torch::Tensor router_w,
 
 std::vector<torch::Tensor> moe_route_all(torch::Tensor h, torch::Tensor router_w,
                                          c10::optional<torch::Tensor> correction,
-                                         int64_t top, double scale) {
-  return moe_route_impl(h, router_w, c10::nullopt, top, true, correction, scale);
+                                         int64_t top, double scale, int64_t groups,
+                                         int64_t keep_groups, bool renorm) {
+  return moe_route_impl(h, router_w, c10::nullopt, top, true, correction, scale, false, groups,
+                        keep_groups, renorm);
 }
 
 std::vector<torch::Tensor> moe_route_sigmoid(torch::Tensor h, torch::Tensor router_w,
@@ -599,15 +642,17 @@ std::vector<torch::Tensor> moe_route_sigmoid(torch::Tensor h, torch::Tensor rout
 
 static torch::Tensor moe_experts_impl(torch::Tensor h, torch::Tensor idx, torch::Tensor wts,
                                       torch::Tensor exp_gu, torch::Tensor exp_down, float limit,
-                                      bool scale_input = false) {
+                                      bool scale_input = false, bool relu2 = false) {
   SM_CHECK_CUDA(h); SM_CHECK_CUDA(idx); SM_CHECK_I32(idx); SM_CHECK_CUDA(wts); SM_CHECK_F32(wts);
   SM_CHECK_CUDA(exp_gu); SM_CHECK_CUDA(exp_down);
   const int64_t T = h.size(0);
   const int D = h.size(1);
   const int top = idx.size(1);
   const int E = exp_gu.size(0);
-  const int ff = exp_gu.size(1) / 2;
-  TORCH_CHECK(exp_gu.dim() == 3 && exp_gu.size(1) == 2 * ff && exp_gu.size(2) == D, "moe_experts: gate/up shape");
+  TORCH_CHECK(exp_gu.dim() == 3 && exp_down.dim() == 3, "moe_experts: weights");
+  const int ff = exp_down.size(2);         // relu2: one input matrix, else [gate; up]
+  TORCH_CHECK(exp_gu.size(1) == (relu2 ? ff : 2 * ff) && exp_gu.size(2) == D,
+              "moe_experts: gate/up shape");
   TORCH_CHECK(exp_down.dim() == 3 && exp_down.size(0) == E && exp_down.size(1) == D &&
               exp_down.size(2) == ff, "moe_experts: down shape");
   TORCH_CHECK(idx.size(0) == T && wts.size(0) == T && wts.size(1) == top, "moe_experts: routing shape");
@@ -643,7 +688,8 @@ static torch::Tensor moe_experts_impl(torch::Tensor h, torch::Tensor idx, torch:
     if (M <= 16 * E) {
       // a few rows per expert (decoding): 16x16 tiles, K split over four waves
       const int row_tiles = SM_CDIV(M, 16) + E;
-      moe_gemm_bf16_splitk_kernel<0><<<dim3(row_tiles, SM_CDIV(ff, 16)), 256, 0, stream>>>(
+      auto up = relu2 ? moe_gemm_bf16_splitk_kernel<2> : moe_gemm_bf16_splitk_kernel<0>;
+      up<<<dim3(row_tiles, SM_CDIV(ff, 16)), 256, 0, stream>>>(
           hp, src.data_ptr<int>(), gup, off.data_ptr<int>(), E, ff, D, act.data_ptr(), limit, rw);
       SM_CHECK_LAUNCH();
       moe_gemm_bf16_splitk_kernel<1><<<dim3(row_tiles, SM_CDIV(D, 16)), 256, 0, stream>>>(
@@ -652,7 +698,8 @@ static torch::Tensor moe_experts_impl(torch::Tensor h, torch::Tensor idx, torch:
       SM_CHECK_LAUNCH();
     } else {
       const int row_tiles = SM_CDIV(M, 64) + E;
-      moe_gemm_bf16_kernel<0, 4, 4><<<dim3(row_tiles, SM_CDIV(ff, 64)), 256, 0, stream>>>(
+      auto up = relu2 ? moe_gemm_bf16_kernel<2, 4, 4> : moe_gemm_bf16_kernel<0, 4, 4>;
+      up<<<dim3(row_tiles, SM_CDIV(ff, 64)), 256, 0, stream>>>(
           hp, src.data_ptr<int>(), gup, off.data_ptr<int>(), E, ff, D, act.data_ptr(), limit, rw);
       SM_CHECK_LAUNCH();
       moe_gemm_bf16_kernel<1, 4, 4><<<dim3(row_tiles, SM_CDIV(D, 64)), 256, 0, stream>>>(
@@ -663,7 +710,8 @@ static torch::Tensor moe_experts_impl(torch::Tensor h, torch::Tensor idx, torch:
   } else {
     SM_CHECK_F32(h);
     auto act = torch::empty({M, ff}, h.options());
-    moe_gemm_f32_kernel<0><<<SM_CDIV(M * ff, 256), 256, 0, stream>>>(
+    auto up = relu2 ? moe_gemm_f32_kernel<2> : moe_gemm_f32_kernel<0>;
+    up<<<SM_CDIV(M * ff, 256), 256, 0, stream>>>(
         h.data_ptr<float>(), src.data_ptr<int>(), exp_gu.data_ptr<float>(),
         off.data_ptr<int>(), E, (int)M, ff, D, act.data_ptr<float>(), limit, rw);
     SM_CHECK_LAUNCH();
@@ -699,4 +747,9 @@ torch::Tensor moe_experts_glu(torch::Tensor h, torch::Tensor idx, torch::Tensor 
 torch::Tensor moe_experts_scaled_input(torch::Tensor h, torch::Tensor idx, torch::Tensor wts,
                                        torch::Tensor exp_gu, torch::Tensor exp_down) {
   return moe_experts_impl(h, idx, wts, exp_gu, exp_down, 0.f, true);
+}
+
+torch::Tensor moe_experts_relu2(torch::Tensor h, torch::Tensor idx, torch::Tensor wts,
+                                torch::Tensor exp_up, torch::Tensor exp_down) {
+  return moe_experts_impl(h, idx, wts, exp_up, exp_down, 0.f, false, true);
 }

@@ -59,6 +59,48 @@ SM_INLINE float sm_block_sum(float x, float* red) {
   return r;
 }
 SM_INLINE float sm_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+// 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))), fp32 inside.
+SM_INLINE float gelu_tanh_f(float z) {
+  return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
+// VEC (1 or 4) neighbouring row entries as fp32, one access each.
+template <int VEC> struct sm_vec { float v[VEC]; };
+
+template <int VEC> SM_INLINE sm_vec<VEC> sm_load(const float* p) {
+  sm_vec<VEC> r;
+  if constexpr (VEC == 4) {
+    const float4 a = *reinterpret_cast<const float4*>(p);
+    r.v[0] = a.x; r.v[1] = a.y; r.v[2] = a.z; r.v[3] = a.w;
+  } else {
+    r.v[0] = *p;
+  }
+  return r;
+}
+template <int VEC> SM_INLINE sm_vec<VEC> sm_load(const bf16_t* p) {
+  sm_vec<VEC> r;
+  if constexpr (VEC == 4) {
+    const uint2 a = *reinterpret_cast<const uint2*>(p);
+    r.v[0] = __uint_as_float(a.x << 16); r.v[1] = __uint_as_float(a.x & 0xffff0000u);
+    r.v[2] = __uint_as_float(a.y << 16); r.v[3] = __uint_as_float(a.y & 0xffff0000u);
+  } else {
+    r.v[0] = to_f(*p);
+  }
+  return r;
+}
+template <int VEC> SM_INLINE void sm_store(float* p, const sm_vec<VEC>& r) {
+  if constexpr (VEC == 4) *reinterpret_cast<float4*>(p) = make_float4(r.v[0], r.v[1], r.v[2], r.v[3]);
+  else *p = r.v[0];
+}
+template <int VEC> SM_INLINE void sm_store(bf16_t* p, const sm_vec<VEC>& r) {
+  if constexpr (VEC == 4) {
+    unsigned int w[4];
+    #pragma unroll
+    for (int k = 0; k < 4; ++k) w[k] = __bfloat16_as_ushort(__float2bfloat16(r.v[k]));
+    *reinterpret_cast<uint2*>(p) = make_uint2(w[0] | (w[1] << 16), w[2] | (w[3] << 16));
+  } else {
+    *p = __float2bfloat16(r.v[0]);
+  }
+}
 // Differential attention: lam_w = lq1 | lk1 | lq2 | lk2 (dk entries each);
 // lambda = exp(lq1.lk1) - exp(lq2.lk2) + diff, the difference's norm takes eps.
 struct wa_diff {
@@ -73,6 +115,25 @@ SM_INLINE float wa_lambda(const wa_diff& df, int dk, int lane) {
     s2 = fmaf(df.lam_w[2 * dk + k], df.lam_w[3 * dk + k], s2);
   }
   return expf(sm_wave_sum(s1)) - expf(sm_wave_sum(s2)) + df.diff;
+}
+// Which keys a query sees besides j <= p: the last `window` positions (0: all),
+// its own chunk of `chunk` positions (0: no chunks) and the first `keep` tokens;
+// how its scores close: cap tanh(score / cap) (0: as they are) and a per-head
+// sink that joins the softmax denominator (null: none).
+struct wa_view {
+  int window, chunk, keep;
+  float cap;
+  const float* sink;
+};
+// First position of the range that ends at p.
+SM_INLINE int wa_first(const wa_view& v, int p) {
+  int lo = (v.window > 0 && p - v.window + 1 > 0) ? p - v.window + 1 : 0;
+  if (v.chunk > 0) lo = max(lo, p / v.chunk * v.chunk);
+  return lo;
+}
+// What the sink adds to a softmax sum taken relative to the maximum m.
+SM_INLINE float wa_sink(const wa_view& v, int head, float m) {
+  return v.sink != nullptr ? expf(v.sink[head] - m) : 0.f;
 }
 // clamped GLU: g = min(gate, limit), u = clamp(up, +-limit), g sigmoid(1.702 g) (u + 1)
 SM_INLINE float sm_capped_glu(float g, float u, float limit) {

@@ -3,8 +3,9 @@
 // RMS-normed q/k heads (before or after the rotation), half-layout rotary from
 // a frequency table, queries scaled with their position, scores mixed across
 // heads before the softmax, a logarithmic distance bias, a window that keeps
-// the first tokens, two maps per head over the same values (differential
-// attention) and a sigmoid output gate per head or per entry.
+// the first tokens or chunks a query does not see beyond, two maps per head over
+// the same values (differential attention), tanh-capped scores, a per-head sink
+// in the softmax denominator and a sigmoid output gate per head or per entry.
 //
 // Two maps: query head h has the rows (h, map 1), (h, map 2), a kv head two
 // key parts and one value part. The softmaxes of both maps are carried side by
@@ -25,8 +26,9 @@
 //   window_attention        one wave per (token, head): any shape
 // (the tiled MFMA kernel for bf16 prompt portions is in
 // window_attention_mfma.hip)
-// A query at position p sees the keys [0, min(keep, lo)) and [lo, p] with
-// lo = max(0, p - window + 1); the kernels walk the two ranges as one list.
+// A query at position p sees the keys [0, min(keep, lo)) and [lo, p], lo the
+// start of its window or chunk (wa_first); the kernels walk the two ranges as
+// one list.
 #include <torch/extension.h>
 #include <ATen/cuda/CUDAContext.h>
 #include "seqmix_common.h"
@@ -286,7 +288,7 @@ __global__ __launch_bounds__(64) void window_attention_kernel(
     const T* __restrict__ cache,      // [rows, G MAPS dk + G vd]
     const int* __restrict__ block_tables, int max_nb, int block_size,
     const int* __restrict__ tok_seq, const int* __restrict__ positions, int H, int G,
-    int dk, int vd, int whole_key, float scale, int window, int keep,
+    int dk, int vd, int whole_key, float scale, wa_view vw,
     const float* __restrict__ r1, const float* __restrict__ r2,
     const T* __restrict__ gate, int64_t ldg, int gs, wa_diff df,
     T* __restrict__ out) {            // [Tn, H vd]
@@ -299,8 +301,8 @@ __global__ __launch_bounds__(64) void window_attention_kernel(
   const int64_t W = (int64_t)G * (MAPS * dk + vd);
   const int voff = G * MAPS * dk + g * vd;
   const int b = tok_seq[t], p = positions[t];
-  const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
-  const int nfirst = (window > 0) ? min(keep, lo) : 0;
+  const int lo = wa_first(vw, p);
+  const int nfirst = min(vw.keep, lo);
   const int n = nfirst + (p - lo + 1);
   const int* bt = block_tables + (int64_t)b * max_nb;
   const float a1 = (r1 != nullptr) ? r1[hd] : 0.f, a2 = (r1 != nullptr) ? r2[hd] : 0.f;
@@ -328,6 +330,7 @@ __global__ __launch_bounds__(64) void window_attention_kernel(
         float dot = 0.f;
         for (int k = 0; k < KD; ++k) dot = fmaf(qs[k], to_f(kp[k]), dot);
         s = dot * scale;
+        if (vw.cap > 0.f) s = vw.cap * tanhf(s / vw.cap);
         if (r1 != nullptr) s -= wa_bias(a1, a2, p - j);
       }
       const float m_new = fmaxf(m, sm_wave_max(s));    // finite: the list is never empty
@@ -351,6 +354,7 @@ __global__ __launch_bounds__(64) void window_attention_kernel(
         }
       }
     }
+    l[mp] += wa_sink(vw, hd, m);
   }
   float o[WA_REGS], f = 1.0f;
   if (MAPS == 2) {
@@ -396,7 +400,7 @@ __global__ __launch_bounds__(256) void window_attention_group_kernel(
     const T* __restrict__ cache,      // [rows, G MAPS dk + G vd]
     const int* __restrict__ block_tables, int max_nb, int block_size,
     const int* __restrict__ tok_seq, const int* __restrict__ positions, int H, int G,
-    int dk, int vd, int whole_key, float scale, int window, int keep,
+    int dk, int vd, int whole_key, float scale, wa_view vw,
     const float* __restrict__ r1, const float* __restrict__ r2,
     const T* __restrict__ gate, int64_t ldg, int gs, wa_diff df, int ksplit,
     float* __restrict__ part,         // [ksplit, Tn, H MAPS, vd] when ksplit > 1
@@ -418,8 +422,8 @@ __global__ __launch_bounds__(256) void window_attention_group_kernel(
   for (int i = tid; i < VR * KD; i += 256)
     qs[i] = to_f(q[((int64_t)t * HV + h0 * MAPS + i / KD) * KD + i % KD]);
   const int b = tok_seq[t], p = positions[t];
-  const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
-  const int nfirst = (window > 0) ? min(keep, lo) : 0;
+  const int lo = wa_first(vw, p);
+  const int nfirst = min(vw.keep, lo);
   const int n = nfirst + (p - lo + 1);
   const int nblk = (n + 63) / 64;
   const int kb_lo = (int)(((int64_t)nblk * z) / ksplit);
@@ -485,6 +489,7 @@ __global__ __launch_bounds__(256) void window_attention_group_kernel(
       float x = -INFINITY;
       if (i < n) {
         x = s[hh] * scale;
+        if (vw.cap > 0.f) x = vw.cap * tanhf(x / vw.cap);
         if (r1 != nullptr) x -= wa_bias(a1[hh / MAPS], a2[hh / MAPS], p - j);
       }
       const float mn = fmaxf(m[hh], sm_wave_max(x));   // finite: the block holds a key
@@ -564,7 +569,8 @@ __global__ __launch_bounds__(256) void window_attention_group_kernel(
         e[w] = (mw == -INFINITY) ? 0.f : expf(mw - M);
         L += red[(w * VR + hv) * RS + vd + 1] * e[w];
       }
-      const float f = (ksplit == 1) ? 1.0f / L : 1.0f;
+      // the sink joins where the softmax is closed: here, or in the merge
+      const float f = (ksplit == 1) ? 1.0f / (L + wa_sink(vw, h0 + hh, M)) : 1.0f;
       const int64_t at = ((int64_t)z * gridDim.x + t) * HV + h0 * MAPS + hv;
       if (ksplit > 1 && lane == 0) {
         part_ml[at * 2] = M;
@@ -624,7 +630,7 @@ template <typename T, int MAPS>
 __global__ __launch_bounds__(64) void window_attention_merge_kernel(
     const float* __restrict__ part, const float* __restrict__ part_ml, int Tn, int H, int vd,
     int ksplit, const T* __restrict__ gate, int64_t ldg, int gs, wa_diff df, int dk,
-    T* __restrict__ out) {
+    wa_view vw, T* __restrict__ out) {
   constexpr int NR = WAG_CP * 2;                     // value entries per lane
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const int64_t stride = (int64_t)Tn * H * MAPS;
@@ -648,8 +654,9 @@ __global__ __launch_bounds__(64) void window_attention_merge_kernel(
         if (d < vd) a[mp][r] += part[(s * stride + th) * vd + d] * e;
       }
     }
+    const float f = 1.0f / (L + wa_sink(vw, h, M));
     #pragma unroll
-    for (int r = 0; r < NR; ++r) a[mp][r] *= 1.0f / L;
+    for (int r = 0; r < NR; ++r) a[mp][r] *= f;
   }
   float post = 1.0f;
   if (MAPS == 2) {
@@ -675,9 +682,10 @@ __global__ __launch_bounds__(64) void window_attention_merge_kernel(
 
 // What the attention kernels are called with.
 struct wa_args {
-  int KD, max_nb, block_size, H, G, dk, vd, whole, window, keep, gs, maps;
+  int KD, max_nb, block_size, H, G, dk, vd, whole, gs, maps;
   const int *bt, *tok_seq, *pos;
   float scale;
+  wa_view vw;
   const float *r1, *r2;
   const void* gate;
   int64_t ldg;
@@ -702,8 +710,8 @@ bool launch_group(int rep, dim3 grid, size_t lds, hipStream_t stream, const T* q
       raised = (int)lds;                                                                     \
     }                                                                                        \
     kern<<<grid, 256, lds, stream>>>(q, a.KD, cache, a.bt, a.max_nb, a.block_size, a.tok_seq, \
-                                     a.pos, a.H, a.G, a.dk, a.vd, a.whole, a.scale, a.window, \
-                                     a.keep, a.r1, a.r2, reinterpret_cast<const T*>(a.gate),  \
+                                     a.pos, a.H, a.G, a.dk, a.vd, a.whole, a.scale, a.vw, \
+                                     a.r1, a.r2, reinterpret_cast<const T*>(a.gate),  \
                                      a.ldg, a.gs, a.df, ksplit, part, part_ml, out);         \
     return true;                                                                             \
   }
@@ -726,7 +734,9 @@ void run_plain(torch::Tensor& q, torch::Tensor& cache, const wa_args& a, bool gr
     const size_t lds = wag_lds_bytes(rep * a.maps, a.KD, a.vd);
     // enough key shares to fill the chip, at least four 64-key blocks each;
     // from host-side sizes only, so a captured step keeps its grid
-    const int64_t longest = (a.window > 0) ? a.window + a.keep : (int64_t)a.max_nb * a.block_size;
+    int64_t longest = (int64_t)a.max_nb * a.block_size;
+    if (a.vw.window > 0) longest = std::min<int64_t>(longest, a.vw.window + a.vw.keep);
+    if (a.vw.chunk > 0) longest = std::min<int64_t>(longest, a.vw.chunk + a.vw.keep);
     int ksplit = (int)std::min<int64_t>(std::max<int64_t>(1, 512 / std::max<int64_t>(1, Tn * a.G)),
                                         std::max<int64_t>(1, longest / 256));
     ksplit = std::min(ksplit, 16);
@@ -747,10 +757,10 @@ void run_plain(torch::Tensor& q, torch::Tensor& cache, const wa_args& a, bool gr
     if (ksplit > 1) {
       if (a.maps == 2)
         window_attention_merge_kernel<T, 2><<<dim3(Tn, a.H), 64, 0, stream>>>(
-            pp, pm, (int)Tn, a.H, a.vd, ksplit, gp, a.ldg, a.gs, a.df, a.dk, op);
+            pp, pm, (int)Tn, a.H, a.vd, ksplit, gp, a.ldg, a.gs, a.df, a.dk, a.vw, op);
       else
         window_attention_merge_kernel<T, 1><<<dim3(Tn, a.H), 64, 0, stream>>>(
-            pp, pm, (int)Tn, a.H, a.vd, ksplit, gp, a.ldg, a.gs, a.df, a.dk, op);
+            pp, pm, (int)Tn, a.H, a.vd, ksplit, gp, a.ldg, a.gs, a.df, a.dk, a.vw, op);
       SM_CHECK_LAUNCH();
     }
     return;
@@ -759,7 +769,7 @@ void run_plain(torch::Tensor& q, torch::Tensor& cache, const wa_args& a, bool gr
 #define WA_PLAIN(M)                                                                          \
   window_attention_kernel<T, M><<<dim3(Tn, a.H), 64, lds, stream>>>(                         \
       qp, a.KD, cp, a.bt, a.max_nb, a.block_size, a.tok_seq, a.pos, a.H, a.G, a.dk, a.vd,    \
-      a.whole, a.scale, a.window, a.keep, a.r1, a.r2, gp, a.ldg, a.gs, a.df, op)
+      a.whole, a.scale, a.vw, a.r1, a.r2, gp, a.ldg, a.gs, a.df, op)
   if (a.maps == 2) WA_PLAIN(2); else WA_PLAIN(1);
 #undef WA_PLAIN
   SM_CHECK_LAUNCH();
@@ -892,10 +902,10 @@ torch::Tensor qk_prepare_kv_write(torch::Tensor proj, int64_t heads, int64_t kv_
 }
 
 // defined in window_attention_mfma.hip
-bool window_attention_mfma_fits(int KD, int vd, int maps);
+bool window_attention_mfma_fits(int KD, int vd, int maps, bool dist, bool cap);
 void window_attention_mfma(torch::Tensor q, int KD, torch::Tensor cache, int H, int G, int dk, int vd,
                            int whole_key, torch::Tensor block_tables, int block_size,
-                           torch::Tensor positions, float scale, int window, int keep,
+                           torch::Tensor positions, float scale, wa_view vw,
                            const float* r1, const float* r2, const void* gate, int64_t ldg, int gs,
                            int maps, wa_diff df, torch::Tensor tiles, torch::Tensor out);
 
@@ -908,7 +918,8 @@ torch::Tensor window_attention(torch::Tensor q, torch::Tensor cache, int64_t hea
                                c10::optional<torch::Tensor> gate,
                                c10::optional<torch::Tensor> tiles, int64_t max_tile_queries,
                                int64_t maps, c10::optional<torch::Tensor> lam_w, double diff,
-                               double eps) {
+                               double eps, int64_t chunk, double softcap,
+                               c10::optional<torch::Tensor> sink) {
   SM_CHECK_CUDA(q); SM_CHECK_CUDA(cache); SM_CHECK_CUDA(block_tables); SM_CHECK_I32(block_tables);
   SM_CHECK_CUDA(tok_seq); SM_CHECK_I32(tok_seq); SM_CHECK_CUDA(positions); SM_CHECK_I32(positions);
   const int H = heads, G = kv_heads, dk = dim, vd = vdim, MP = maps;
@@ -925,7 +936,8 @@ torch::Tensor window_attention(torch::Tensor q, torch::Tensor cache, int64_t hea
   TORCH_CHECK(block_tables.dim() == 2 && tok_seq.numel() == T && positions.numel() == T &&
               block_size > 0, "window_attention: batch layout");
   TORCH_CHECK(vd >= 1 && vd <= 64 * WA_REGS, "window_attention: value size above 512");
-  TORCH_CHECK(window >= 0 && keep_first >= 0, "window_attention: window");
+  TORCH_CHECK(window >= 0 && keep_first >= 0 && chunk >= 0 && softcap >= 0.0,
+              "window_attention: window, chunk, cap");
   TORCH_CHECK(r1.has_value() == r2.has_value(), "window_attention: both distance factors or none");
   wa_args a = {};
   if (r1.has_value()) {
@@ -951,7 +963,13 @@ torch::Tensor window_attention(torch::Tensor q, torch::Tensor cache, int64_t hea
     a.df = {lam_w->data_ptr<float>(), (float)diff, (float)eps};
   }
   a.KD = KD; a.max_nb = block_tables.size(1); a.block_size = block_size; a.H = H; a.G = G;
-  a.dk = dk; a.vd = vd; a.whole = whole_key ? 1 : 0; a.window = window; a.keep = keep_first;
+  a.dk = dk; a.vd = vd; a.whole = whole_key ? 1 : 0;
+  a.vw = {(int)window, (int)chunk, (int)keep_first, (float)softcap, nullptr};
+  if (sink.has_value()) {
+    SM_CHECK_CUDA(*sink); SM_CHECK_F32(*sink);
+    TORCH_CHECK(sink->numel() == H, "window_attention: one sink per head");
+    a.vw.sink = sink->data_ptr<float>();
+  }
   a.maps = MP; a.bt = block_tables.data_ptr<int>(); a.tok_seq = tok_seq.data_ptr<int>();
   a.pos = positions.data_ptr<int>(); a.scale = scale;
   auto out = torch::empty({T, (int64_t)H * vd}, q.options());
@@ -960,12 +978,12 @@ torch::Tensor window_attention(torch::Tensor q, torch::Tensor cache, int64_t hea
   const bool is_bf16 = q.scalar_type() == at::kBFloat16;
   if (!is_bf16) SM_CHECK_F32(q);
   if (is_bf16 && tiles.has_value() && max_tile_queries > 4 &&
-      window_attention_mfma_fits(KD, vd, MP)) {
+      window_attention_mfma_fits(KD, vd, MP, r1.has_value(), softcap > 0.0)) {
     SM_CHECK_CUDA(*tiles); SM_CHECK_I32(*tiles);
     TORCH_CHECK(tiles->dim() == 2 && tiles->size(1) == 3 && max_tile_queries <= 64,
                 "window_attention: tiles");
     window_attention_mfma(q, KD, cache, H, G, dk, vd, a.whole, block_tables, (int)block_size,
-                          positions, a.scale, a.window, a.keep, a.r1, a.r2, a.gate, a.ldg, a.gs, MP,
+                          positions, a.scale, a.vw, a.r1, a.r2, a.gate, a.ldg, a.gs, MP,
                           a.df, *tiles, out);
     return out;
   }

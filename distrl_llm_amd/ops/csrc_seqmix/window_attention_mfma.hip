@@ -11,8 +11,8 @@
 // (transposed) are staged in LDS once per tile.
 //   scores   MFMA 16x16x32: A = the wave's queries (registers, loaded once),
 //            B = K rows from LDS
-//   softmax  fp32 in the MFMA's result layout; distance bias and mask per
-//            score; row reductions over the 16 lanes of a row by lane
+//   softmax  fp32 in the MFMA's result layout; cap, distance bias and mask per
+//            score, the sink where the sum is closed; row reductions over the 16 lanes of a row by lane
 //            permutes. The distance bias depends on (head, distance) only and
 //            a wave's 16 queries meet a block's keys at KB + 15 distances:
 //            the wave tabulates those once per block instead of taking a
@@ -36,18 +36,24 @@ typedef __attribute__((ext_vector_type(4))) float f32x4;
 
 namespace {
 
+// cap tanh(x / cap), tanh z = 1 - 2 / (1 + e^(2z)): absolute error of a few
+// fp32 roundings of cap; saturates to +-cap.
+SM_INLINE float wam_cap(float x, float cap, float icap) {
+  return cap - 2.0f * cap / (1.0f + __expf(2.0f * x * icap));
+}
+
 // NT: 16-column value tiles per wave (vd <= 16 NT); KS: 32-entry steps of the
 // query/key dot product held in registers (KD <= 32 KS); KB: keys per block;
 // DIST: the distance bias is taken off the scores (r1, r2 given); MAPS: query
-// and key maps per head.
-template <int NT, int KS, int KB, bool DIST, int MAPS>
+// and key maps per head; CAP: scores become cap tanh(score / cap).
+template <int NT, int KS, int KB, bool DIST, int MAPS, bool CAP>
 __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
     const bf16_t* __restrict__ q, int KD,  // [Tn, H MAPS, KD]
     const bf16_t* __restrict__ cache,      // [rows, G (MAPS dk + vd)]
     const int* __restrict__ block_tables, int max_nb, int block_size,
     const int* __restrict__ positions,
     const int* __restrict__ tiles,         // [ntiles, 3] = (batch row, first token, queries)
-    int H, int G, int dk, int vd, int whole_key, float scale, int window, int keep,
+    int H, int G, int dk, int vd, int whole_key, float scale, wa_view vw,
     const float* __restrict__ r1, const float* __restrict__ r2,
     const bf16_t* __restrict__ gate, int64_t ldg, int gs, wa_diff df,
     bf16_t* __restrict__ out) {            // [Tn, H vd]
@@ -73,14 +79,15 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
   const int grp = hd / (H / G);
   const int koff = whole_key ? 0 : grp * MAPS * dk, voff = G * MAPS * dk + grp * vd;
   const int p0 = positions[t0], plast = p0 + nq - 1;
-  const int lo = (window > 0 && p0 - window + 1 > 0) ? p0 - window + 1 : 0;
-  const int nf = (window > 0) ? min(keep, lo) : 0; // kept keys before the first window
+  const int lo = wa_first(vw, p0);
+  const int nf = min(vw.keep, lo);                 // kept keys before the first window or chunk
   const int n = nf + (plast - lo + 1);             // keys in the tile's list
   const int nblk = (n + WAM_KB - 1) / WAM_KB;
   const int* bt = block_tables + (int64_t)b * max_nb;
   float* p_lds = p_all + wave * 16 * WAM_PP;
   float* tb = tb_all + wave * WAM_TB;
   const bool active = wave * 16 < nq;
+  const float icap = CAP ? 1.0f / vw.cap : 0.f;
   const float a1 = DIST ? r1[hd] : 0.f, a2 = DIST ? r2[hd] : 0.f;
 
   // the wave's queries as A fragments: row lrow, k = ks * 32 + lk * 8 ..
@@ -100,6 +107,9 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
   // padding rows of v_lds (value columns vd .. NVp) stay zero
   for (int i = tid; i < (NVp - vd) * WAM_VP; i += 256) v_lds[vd * WAM_VP + i] = __float2bfloat16(0.f);
 
+  int first[4];                                    // where each of the lane's queries starts to see
+  #pragma unroll
+  for (int r = 0; r < 4; ++r) first[r] = wa_first(vw, p0 + min(wave * 16 + lk * 4 + r, nq - 1));
   float m[MAPS][4], lsum[MAPS][4];
   f32x4 acc[MAPS][NT];
   #pragma unroll
@@ -150,7 +160,7 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
       const int jb0 = lo + (i0 - nf);
       const int wq_last = min(plast, p0 + wave * 16 + 15), wq_first = p0 + wave * 16;
       if (jb0 > wq_last) continue;
-      if (window > 0 && jb0 + WAM_KB - 1 < wq_first - window + 1 && jb0 >= keep) continue;
+      if (jb0 + WAM_KB - 1 < wa_first(vw, wq_first) && jb0 >= vw.keep) continue;
     }
 
     // distance bias of this wave and block: the block's keys are consecutive
@@ -193,8 +203,9 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
         for (int ct = 0; ct < KB / 16; ++ct) {
           const int i = i0 + ct * 16 + lrow;
           const int j = (i < nf) ? i : lo + (i - nf);
-          const bool seen = i < n && j <= prow && (window <= 0 || prow - j < window || j < keep);
+          const bool seen = i < n && j <= prow && (j >= first[r] || j < vw.keep);
           float x = s[ct][r] * scale;
+          if (CAP) x = wam_cap(x, vw.cap, icap);
           if (DIST) {
             if (tabled) x -= tb[lk * 4 + r + (KB - 1) - (ct * 16 + lrow)];
             else if (seen) x -= a1 * log1pf(a2 * (float)(prow - j));
@@ -260,10 +271,10 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
   #pragma unroll
   for (int r = 0; r < 4; ++r) {
     const int qi = wave * 16 + lk * 4 + r;
-    float f = 1.0f / lsum[0][r];
+    float f = 1.0f / (lsum[0][r] + wa_sink(vw, hd, m[0][r]));
     if (MAPS == 2) {
       // the difference replaces map 1's sums; columns past vd hold zeros
-      const float f2 = lam / lsum[MAPS - 1][r];
+      const float f2 = lam / (lsum[MAPS - 1][r] + wa_sink(vw, hd, m[MAPS - 1][r]));
       float ss = 0.f;
       #pragma unroll
       for (int nt = 0; nt < NT; ++nt) {
@@ -302,14 +313,15 @@ size_t wam_lds_bytes(int KD, int vd, bool dist, int maps) {
 
 // 16-byte pieces of the cache rows: the key columns a head meets (dim, or
 // kv_heads * dim for folded queries) and the value size are multiples of 8
-bool window_attention_mfma_fits(int KD, int vd, int maps) {
-  return KD % 8 == 0 && vd % 8 == 0 && KD <= (maps == 2 ? 128 : 512) && vd <= 256 &&
+bool window_attention_mfma_fits(int KD, int vd, int maps, bool dist, bool cap) {
+  return !(cap && (dist || maps == 2)) && KD % 8 == 0 && vd % 8 == 0 &&
+         KD <= (maps == 2 ? 128 : 512) && vd <= 256 &&
          wam_lds_bytes(KD, vd, true, maps) <= 150 * 1024;
 }
 
 void window_attention_mfma(torch::Tensor q, int KD, torch::Tensor cache, int H, int G, int dk, int vd,
                            int whole_key, torch::Tensor block_tables, int block_size,
-                           torch::Tensor positions, float scale, int window, int keep,
+                           torch::Tensor positions, float scale, wa_view vw,
                            const float* r1, const float* r2, const void* gate, int64_t ldg, int gs,
                            int maps, wa_diff df, torch::Tensor tiles, torch::Tensor out) {
   const int ntiles = tiles.size(0);
@@ -317,9 +329,9 @@ void window_attention_mfma(torch::Tensor q, int KD, torch::Tensor cache, int H, 
   auto stream = at::cuda::getCurrentCUDAStream();
   const size_t lds = wam_lds_bytes(KD, vd, r1 != nullptr, maps);
   dim3 grid(ntiles, H);
-#define WAM_LAUNCH(NT, KS, DIST, MAPS)                                                         \
+#define WAM_LAUNCH(NT, KS, DIST, MAPS, CAP)                                                       \
   do {                                                                                         \
-    auto kern = window_attention_mfma_kernel<NT, KS, WAM_KEYS, DIST, MAPS>;                    \
+    auto kern = window_attention_mfma_kernel<NT, KS, WAM_KEYS, DIST, MAPS, CAP>;                  \
     static int raised = 0;                                                                     \
     if (lds > 64 * 1024 && (int)lds > raised) {                                                \
       TORCH_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(kern),                     \
@@ -331,20 +343,20 @@ void window_attention_mfma(torch::Tensor q, int KD, torch::Tensor cache, int H, 
         reinterpret_cast<const bf16_t*>(q.data_ptr()), KD,                                     \
         reinterpret_cast<const bf16_t*>(cache.data_ptr()), block_tables.data_ptr<int>(),       \
         (int)block_tables.size(1), block_size, positions.data_ptr<int>(), tiles.data_ptr<int>(), \
-        H, G, dk, vd, whole_key, scale, window, keep, r1, r2,                                  \
+        H, G, dk, vd, whole_key, scale, vw, r1, r2,                                            \
         reinterpret_cast<const bf16_t*>(gate), ldg, gs, df,                                    \
         reinterpret_cast<bf16_t*>(out.data_ptr()));                                            \
   } while (0)
-#define WAM_BY_KS(NT, DIST)                                  \
+#define WAM_BY_KS(NT, DIST, CAP)                             \
   do {                                                       \
-    if (KD <= 128) WAM_LAUNCH(NT, 4, DIST, 1);               \
-    else if (KD <= 256) WAM_LAUNCH(NT, 8, DIST, 1);          \
-    else WAM_LAUNCH(NT, 16, DIST, 1);                        \
+    if (KD <= 128) WAM_LAUNCH(NT, 4, DIST, 1, CAP);          \
+    else if (KD <= 256) WAM_LAUNCH(NT, 8, DIST, 1, CAP);     \
+    else WAM_LAUNCH(NT, 16, DIST, 1, CAP);                   \
   } while (0)
 #define WAM_BY_KS2(NT)                                       \
   do {                                                       \
-    if (KD <= 64) WAM_LAUNCH(NT, 2, false, 2);               \
-    else WAM_LAUNCH(NT, 4, false, 2);                        \
+    if (KD <= 64) WAM_LAUNCH(NT, 2, false, 2, false);        \
+    else WAM_LAUNCH(NT, 4, false, 2, false);                 \
   } while (0)
 #define WAM_BY_NT(BY, ...)                                   \
   do {                                                       \
@@ -352,9 +364,12 @@ void window_attention_mfma(torch::Tensor q, int KD, torch::Tensor cache, int H, 
     else if (vd <= 128) BY(8, ##__VA_ARGS__);                \
     else BY(16, ##__VA_ARGS__);                              \
   } while (0)
+  // capped scores: one map without distance bias (the caller sends the rest of
+  // the combinations to the other kernels)
   if (maps == 2) WAM_BY_NT(WAM_BY_KS2);
-  else if (r1 != nullptr) WAM_BY_NT(WAM_BY_KS, true);
-  else WAM_BY_NT(WAM_BY_KS, false);
+  else if (r1 != nullptr) WAM_BY_NT(WAM_BY_KS, true, false);
+  else if (vw.cap > 0.f) WAM_BY_NT(WAM_BY_KS, false, true);
+  else WAM_BY_NT(WAM_BY_KS, false, false);
 #undef WAM_BY_NT
 #undef WAM_BY_KS2
 #undef WAM_BY_KS

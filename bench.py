@@ -51,12 +51,12 @@ def parse_args():
                         "no-EOS rounds). Measures in-wave retirement.")
     p.add_argument("--hybrid-bench", type=str, default="",
                    help="instead of the RL round: prefill/decode tokens/s of "
-                        "the layer-list designs (Sagedra, Legilix, Kakilorn, "
+                        "the layer-list designs (Pedazen, Sagedra, Legilix, Kakilorn, "
                         "Nedasun, Nibalix) beside the "
                         "dense model of equal size, at these comma-separated "
                         "sizes (1k,2k)")
     p.add_argument("--hybrid-only", type=str, default="",
-                   help="with --hybrid-bench: run only these of 'sagedra', 'legilix', "
+                   help="with --hybrid-bench: run only these of 'pedazen', 'sagedra', 'legilix', "
                         "'kakilorn', 'nedasun', 'nibalix', 'dense' "
                         "(comma-separated)")
     p.add_argument("--tiny", action="store_true",

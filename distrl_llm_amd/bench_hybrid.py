@@ -1,5 +1,5 @@
 """Prefill and decode throughput of the layer-list designs (Nibalix,
-Nedasun, Kakilorn, Legilix, Sagedra) beside one another and beside the dense
+Nedasun, Kakilorn, Legilix, Sagedra, Pedazen) beside one another and beside the dense
 transformer of equal size (``bench.py --hybrid-bench``).
 
 All models get random weights at layer sizes that resemble a real model
@@ -180,14 +180,51 @@ def sagedra_bench_config(s: dict) -> dict:
             "width": s["width"]}
 
 
+def pedazen_bench_config(s: dict) -> dict:
+    """Same width, head count and head sizes (128/128, 4 query heads per kv
+    head in attention) as the other designs of the size. Six layers run as
+    eight (layers 1 and 2 twice): linear attention, and pairs of chunked
+    attention (chunks as long as the other designs' windows) beside a linear
+    recurrent unit as wide as the model (blocks of 256 channels, 4 taps);
+    feed-forwards alternate between a dense one as wide as the experts a token
+    uses and the experts of the other designs, in four groups of which two are
+    kept."""
+    kvh = max(1, s["heads"] // 4)
+    dense = {"kind": "dense", "ff": s["top"] * s["ff"]}
+    moe = {"kind": "moe", "expert": {"ff": s["ff"]},
+           "router": {"experts": s["experts"], "top": s["top"],
+                      "groups": {"count": 4, "keep": 2}}}
+    light = {"heads": s["heads"], "dim": 128, "vdim": 128,
+             "decay": [1.0 - 2.0 ** (-2.0 - 6.0 * h / s["heads"])
+                       for h in range(s["heads"])]}
+    left = {"heads": s["heads"], "kv_heads": kvh, "dim": 128, "vdim": 128,
+            "scale": 128 ** -0.5, "softcap": 30.0, "mask": {"size": s["window"]},
+            "rot": {"base": 10000.0, "dims": 64}}
+    right = {"width": s["width"], "blocks": s["width"] // 256, "conv": 4}
+    layers = []
+    for i in range(s["layers"] - 2):
+        mlp = dense if i % 2 == 0 else moe
+        if i % 3 == 2:
+            layers.append({"type": "parallel", "mixer": {"left": left, "right": right},
+                           "mlp": mlp})
+        else:
+            layers.append({"type": "lightning", "mixer": light, "mlp": mlp})
+    return {"architecture": "Pedazen", "embedding": {"scale": 1.0}, "layers": layers,
+            "loop": {"start": 1, "stop": 3, "times": 2}, "norm": {"eps": 1e-5},
+            "vocab": s["vocab"], "width": s["width"]}
+
+
 def _build_hybrid(s, device, max_len, batch, design="nibalix"):
     from .engine.hybrid_engine import HybridEngine
     from .models.hybrid import (HybridLM, kakilorn_spec_from_config,
                                 legilix_spec_from_config,
                                 nedasun_spec_from_config,
                                 nibalix_spec_from_config,
+                                pedazen_spec_from_config,
                                 sagedra_spec_from_config)
-    if design == "sagedra":
+    if design == "pedazen":
+        spec = pedazen_spec_from_config(pedazen_bench_config(s))
+    elif design == "sagedra":
         spec = sagedra_spec_from_config(sagedra_bench_config(s))
     elif design == "legilix":
         spec = legilix_spec_from_config(legilix_bench_config(s))
@@ -244,7 +281,7 @@ def measure(engine, vocab, batch, prompt_len, new_tokens, device):
 
 
 def run(sizes, device, batch=16, prompt_len=1024, new_tokens=33,
-        which=("sagedra", "legilix", "kakilorn", "nedasun", "nibalix", "dense")):
+        which=("pedazen", "sagedra", "legilix", "kakilorn", "nedasun", "nibalix", "dense")):
     out = []
     for name in sizes:
         s = SIZES[name]

@@ -227,3 +227,104 @@ def forward(cfg, w, tokens, layers_out=None):
         if layers_out is not None:
             layers_out.append(x)
     return block_norm(x, w["final.norm"].to(F64), eps) @ w["embed"].to(F64).t()
+
+
+# ------------------------------------------------- small configs for tests
+
+def dense(ff=14):
+    return {"kind": "dense", "ff": ff}
+
+
+def moe(experts=6, top=2, ff=10, groups=(3, 2)):
+    rc = {"experts": experts, "top": top}
+    if groups:
+        rc["groups"] = {"count": groups[0], "keep": groups[1]}
+    return {"kind": "moe", "expert": {"ff": ff}, "router": rc}
+
+
+def light_layer(heads=3, dim=6, vdim=10, decay=None, mlp=None):
+    if decay is None:
+        decay = [1.0 - 0.5 * 0.3 ** h for h in range(heads)]
+    return {"type": "lightning", "mlp": mlp,
+            "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "decay": list(decay)}}
+
+
+def pair_layer(heads=4, kv_heads=2, dim=8, vdim=5, chunk=7, rot_dims=6, base=50.0, scale=None,
+               softcap=3.0, width=12, blocks=3, conv=4, mlp=None):
+    left = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim,
+            "rot": {"base": base, "dims": rot_dims}, "mask": {"size": chunk},
+            "scale": scale if scale is not None else dim ** -0.5, "softcap": softcap}
+    return {"type": "parallel", "mlp": mlp,
+            "mixer": {"left": left, "right": {"width": width, "blocks": blocks, "conv": conv}}}
+
+
+def make_cfg(layers, width=20, vocab=37, loop=None, eps=1e-5, embed_scale=3.0):
+    cfg = {"architecture": "Pedazen", "embedding": {"scale": embed_scale}, "layers": layers,
+           "norm": {"eps": eps}, "vocab": vocab, "width": width}
+    if loop:
+        cfg["loop"] = dict(zip(("start", "stop", "times"), loop))
+    return cfg
+
+
+def random_weights(cfg, seed=0):
+    """Checkpoint tensors of a configuration, rounded to bfloat16 as a
+    checkpoint file holds them."""
+    g = torch.Generator().manual_seed(seed)
+    D = int(cfg["width"])
+    w = {}
+
+    def mat(name, rows, cols, gain=1.0):
+        w[name] = gain * torch.randn(rows, cols, generator=g) / math.sqrt(cols)
+
+    def vec(name, n, mean=0.0, std=0.1):
+        w[name] = mean + std * torch.randn(n, generator=g)
+
+    w["embed"] = torch.randn(int(cfg["vocab"]), D, generator=g) * 0.5
+    vec("final.norm", D, 0.0, 0.2)
+    if cfg.get("loop"):
+        w["loop.step"] = 0.7 * torch.randn(int(cfg["loop"]["times"]), D, generator=g)
+    for i, lc in enumerate(cfg["layers"]):
+        p, mc = f"l{i}.", lc["mixer"]
+        x = p + "mix."
+        vec(p + "norm1", D, 0.0, 0.2)
+        if lc["type"] == "lightning":
+            nq, nv = mc["heads"] * mc["dim"], mc["heads"] * mc["vdim"]
+            for nm, rows in (("q", nq), ("k", nq), ("v", nv), ("g", nv)):
+                mat(x + nm, rows, D)
+            vec(x + "norm", nv, 1.0)
+            mat(x + "o", D, nv)
+        else:
+            lm, rm = mc["left"], mc["right"]
+            H, G, dk, dv = lm["heads"], lm["kv_heads"], lm["dim"], lm["vdim"]
+            y = x + "left."
+            for nm, rows in (("q", H * dk), ("k", G * dk), ("v", G * dv)):
+                mat(y + nm, rows, D)
+            vec(y + "q.norm", dk, 1.5, 0.3)
+            vec(y + "k.norm", dk, 1.5, 0.3)
+            vec(y + "sink", H, 0.5, 1.0)
+            mat(y + "o", D, H * dv)
+            vec(y + "out", D, 1.0, 0.2)
+            y, R, B = x + "right.", rm["width"], rm["blocks"]
+            for nm in ("y", "x"):
+                mat(y + nm, R, D)
+                vec(y + nm + ".b", R, 0.0, 0.3)
+            w[y + "conv"] = 0.6 * torch.randn(R, rm["conv"], generator=g)
+            vec(y + "conv.b", R, 0.0, 0.3)
+            for nm in ("ra", "ri"):
+                w[y + nm] = torch.randn(B, R // B, R // B, generator=g) / math.sqrt(R // B)
+                w[y + nm + ".b"] = 0.3 * torch.randn(B, R // B, generator=g)
+            vec(y + "lam", R, -2.5, 1.0)
+            mat(y + "o", D, R)
+            vec(y + "out", D, 1.0, 0.2)
+        f, x = lc.get("mlp"), p + "mlp."
+        if f is not None and f["kind"] == "dense":
+            for nm in ("gate", "up"):
+                mat(x + nm, f["ff"], D)
+            mat(x + "down", D, f["ff"])
+        elif f is not None:
+            # scores well apart: rounding must not change a choice
+            mat(x + "router", f["router"]["experts"], D, 4.0)
+            for e in range(f["router"]["experts"]):
+                mat(f"{x}e{e}.up", f["expert"]["ff"], D)
+                mat(f"{x}e{e}.down", D, f["expert"]["ff"])
+    return {k: v.to(torch.bfloat16).float() for k, v in w.items()}

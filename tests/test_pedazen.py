@@ -1,0 +1,915 @@
+"""Pedazen (parallel block with looped passes, linear attention with fixed
+decays, a normed pair of chunked attention and linear recurrent unit, dense and
+squared-ReLU expert feed-forwards) against the plain oracle in
+pedazen_oracle.py.
+
+Every test builds its own small configuration and random weights. The ``dev``
+fixture runs each case on the CPU path and, marked ``gpu``, on the HIP kernels
+(fp32 and bf16 models).
+"""
+
+import json
+import os
+import subprocess
+import sys
+
+import pytest
+import torch
+
+import pedazen_oracle as O
+from distrl_llm_amd.config import EngineConfig, SamplingParams
+from distrl_llm_amd.engine.hybrid_engine import HybridEngine
+from distrl_llm_amd.models.hybrid import (HybridLM, pedazen_config_from_spec,
+                                          pedazen_spec_from_config,
+                                          rotary_frequencies,
+                                          save_pedazen_checkpoint)
+from distrl_llm_amd.ops import seqmix as SM
+
+CASES = [pytest.param(("cpu", torch.float32), id="cpu-f32"),
+         pytest.param(("cuda", torch.float32), id="gpu-f32", marks=pytest.mark.gpu),
+         pytest.param(("cuda", torch.bfloat16), id="gpu-bf16", marks=pytest.mark.gpu)]
+
+
+@pytest.fixture(params=CASES)
+def dev(request):
+    return request.param
+
+
+def tol(dtype):
+    # whole narrow models in bf16 carry a few percent of rounding noise; the
+    # kernels are held to tighter bounds one by one
+    return 2e-4 if dtype == torch.float32 else 0.1
+
+
+def rel_err(got, want):
+    got, want = got.double().cpu(), want.double().cpu()
+    d = got - want
+    return float(d.pow(2).mean().sqrt() / want.pow(2).mean().sqrt().clamp_min(1e-9))
+
+
+def mixed_cfg():
+    """Both mixers twice, sizes unequal wherever the design allows, dense and
+    expert feed-forwards and a layer without one, the middle layers looped."""
+    return O.make_cfg([
+        O.light_layer(heads=3, dim=6, vdim=10, mlp=O.dense(14)),
+        O.pair_layer(heads=6, kv_heads=2, dim=8, vdim=5, chunk=7, rot_dims=6, width=12, blocks=3,
+                     conv=4, mlp=O.moe(6, 2, 10, (3, 2))),
+        O.light_layer(heads=2, dim=9, vdim=4, decay=[0.3, 0.995], mlp=None),
+        O.pair_layer(heads=2, kv_heads=2, dim=6, vdim=9, chunk=11, rot_dims=6, softcap=20.0,
+                     width=10, blocks=1, conv=2, mlp=O.moe(5, 3, 7, None)),
+    ], width=20, vocab=37, loop=(1, 3, 2))
+
+
+def aligned_cfg():
+    """Sizes the matrix-core kernels take: several 64-token tiles and chunks,
+    more than one block, groups of experts, a loop from layer 0."""
+    return O.make_cfg([
+        O.light_layer(heads=2, dim=40, vdim=48, decay=[0.7, 0.99], mlp=O.moe(8, 3, 24, (4, 2))),
+        O.pair_layer(heads=4, kv_heads=1, dim=24, vdim=16, chunk=50, rot_dims=16, width=80,
+                     blocks=2, conv=4, mlp=O.dense(40)),
+    ], width=32, vocab=41, loop=(0, 1, 2))
+
+
+def build(cfg, dev, seed=0, blocks=64, block_size=4, slots=4, W=None):
+    device, dtype = dev
+    W = W if W is not None else O.random_weights(cfg, seed)
+    model = HybridLM(pedazen_spec_from_config(cfg), dtype=dtype, device=device)
+    model.load_tensors(W)
+    eng = HybridEngine(model, EngineConfig(max_seq_length=4096, kv_block_size=block_size,
+                                           num_kv_blocks=blocks, num_state_slots=slots,
+                                           max_num_seqs=slots), device=torch.device(device))
+    return W, eng
+
+
+def run_portions(eng, tokens, cuts, capture=None):
+    q = eng.open_sequence()
+    out, at = [], 0
+    for n in cuts:
+        out.append(eng.step([(q, tokens[at:at + n])], [list(range(n))], capture=capture))
+        at += n
+    assert at == len(tokens)
+    eng.close_sequence(q)
+    return torch.cat(out)
+
+
+def toks(n, vocab, seed=1):
+    g = torch.Generator().manual_seed(seed)
+    return torch.randint(0, vocab, (n,), generator=g).tolist()
+
+
+def ints(v, device):
+    return torch.tensor(v, dtype=torch.int32, device=device)
+
+
+def layout(lengths, cuts, step, device):
+    """(tokens per row, cu, tok_seq, tiles, tile_cu, max_tile) of one step."""
+    n = [c[step] for c in cuts]
+    cu = [0]
+    for k in n:
+        cu.append(cu[-1] + k)
+    seq = [b for b, k in enumerate(n) for _ in range(k)]
+    tiles, mt = SM.query_tiles(n, SM.WIDE_QUERY_TILE)
+    tc = [0]
+    for k in n:
+        tc.append(tc[-1] + -(-k // SM.WIDE_QUERY_TILE))
+    return n, ints(cu, device), ints(seq, device), ints(tiles, device), ints(tc, device), mt
+
+
+# ------------------------------------------------------ mechanisms alone
+
+@pytest.mark.parametrize("D", [7, 24, 300])
+def test_layer_tail(dev, D):
+    """Start and tail of the parallel block: plain and normed mixer outputs,
+    with and without feed-forward, with nothing, a vector, or vector and
+    embedding row added at the start of a pass, last layer or not."""
+    device, dtype = dev
+    g = torch.Generator().manual_seed(D)
+    T, V, eps = 5, 11, 1e-3
+    embed = torch.randn(V, D, generator=g).to(dtype)
+    ids = torch.tensor([3, 0, 10, 3, 7])
+    nw, lw, rw, step = (0.5 * torch.randn(D, generator=g) for _ in range(4))
+    y, y2, fb = (torch.randn(T, D, generator=g).to(dtype) for _ in range(3))
+    y2 = y2 * 8.0                                   # the sides have unequal sizes
+    f32 = torch.randn(T, D, generator=g)
+    e = embed[ids].double() * 2.5
+    hb_tol = 2e-6 if dtype == torch.float32 else 5e-3
+
+    def to(t):
+        return None if t is None else t.to(device)
+
+    for s in (None, step):
+        x, h = SM.parallel_start(to(embed), to(ids), 2.5, to(s), to(nw), eps, dtype)
+        want = e if s is None else e + s.double()
+        assert rel_err(x, want) < 1e-6 and h.dtype == dtype
+        assert rel_err(h.float(), O.block_norm(want, nw.double(), eps)) < hb_tol
+    x0 = torch.randn(T, D, generator=g)
+    for normed in (False, True):
+        for f in (None, fb, f32):
+            for inj in (None, (None, to(ids), 2.5, to(step)), (to(embed), to(ids), 2.5, to(step))):
+                for last in (False, True):
+                    want = x0.double()
+                    if normed:
+                        want = want + 0.5 * (O.rms_unit(y.double(), eps) * lw.double()
+                                             + O.rms_unit(y2.double(), eps) * rw.double())
+                    else:
+                        want = want + y.double()
+                    if f is not None:
+                        want = want + f.double()
+                    if inj is not None:
+                        want = want + step.double() + (e if inj[0] is not None else 0.0)
+                    x = to(x0.clone())
+                    h = SM.parallel_residual_norm(
+                        x, to(y), to(y2) if normed else None, to(lw) if normed else None,
+                        to(rw) if normed else None, 0.5 if normed else 1.0, 0.5, to(f), inj,
+                        None if last else to(nw), eps, dtype)
+                    assert rel_err(x, want) < 1e-6
+                    assert (h is None) == last
+                    if not last:
+                        assert rel_err(h.float(), O.block_norm(want, nw.double(), eps)) < hb_tol
+
+
+@pytest.mark.parametrize("H,dk,dv,decay", [
+    (3, 6, 10, [0.3, 0.9, 0.999]), (1, 8, 8, [1.0]), (2, 40, 24, [0.5, 0.99]),
+    (4, 72, 8, [0.0, 0.2, 0.97, 0.9995]), (2, 128, 64, [0.8, 0.995]), (1, 3, 1, [0.6]),
+    (2, 200, 40, [0.6, 0.999]), (1, 300, 7, [0.99])])
+def test_linear_attention_op(dev, H, dk, dv, decay):
+    """Two rows of a step cut into portions down to one token (edges of the 64
+    token chunks inside and between portions), scattered slots, strided rows."""
+    device, dtype = dev
+    g = torch.Generator().manual_seed(dk)
+    eps = 1e-4
+    lengths, cuts = [203, 140], [[130, 1, 2, 64, 6], [1, 70, 2, 65, 2]]
+    n = 2 * H * dk + 2 * H * dv
+    full = [torch.randn(L, n + 8, generator=g).to(dtype) for L in lengths]
+    nw = 1.0 + 0.2 * torch.randn(H * dv, generator=g)
+    powers = SM.decay_powers(decay, device)
+    state = torch.zeros(4, H * dv * dk, device=device)
+    slots, got, at = ints([2, 0], device), [[], []], [0, 0]
+    for s in range(5):
+        m, cu, _, _, _, mt = layout(lengths, cuts, s, device)
+        proj = torch.cat([full[b][at[b]:at[b] + m[b]] for b in (0, 1)]).to(device)[:, :n]
+        o = SM.linear_attention(proj, H, dk, dv, powers, nw.to(device), eps, state, cu, slots,
+                                dtype, max_tile=mt)
+        got[0].append(o[:m[0]])
+        got[1].append(o[m[0]:])
+        at = [a + k for a, k in zip(at, m)]
+    assert float(state[1].abs().max()) == 0.0 and float(state[3].abs().max()) == 0.0
+    for b in (0, 1):
+        x = full[b][:, :n].double()
+        q, k = (O.silu(x[:, a * H * dk:(a + 1) * H * dk]).view(-1, H, dk) for a in (0, 1))
+        v = O.silu(x[:, 2 * H * dk:2 * H * dk + H * dv]).view(-1, H, dv)
+        o = O.linear_attention(q, k, v, decay).reshape(lengths[b], -1)
+        o = O.rms_unit(o, eps) * nw.double() * torch.sigmoid(x[:, n - H * dv:])
+        assert rel_err(torch.cat(got[b]).float(), o) < (1e-5 if dtype == torch.float32 else 8e-3)
+
+
+@pytest.mark.parametrize("W,blocks,taps", [(12, 3, 4), (10, 1, 2), (64, 2, 4), (144, 1, 4),
+                                           (48, 6, 3), (320, 2, 1), (8, 8, 5), (16, 2, 4)])
+def test_linear_unit_op(dev, W, blocks, taps):
+    """As above for the recurrent unit: convolution tails over portions shorter
+    than the taps, one block and many, slow and fast channels."""
+    device, dtype = dev
+    g = torch.Generator().manual_seed(W + taps)
+    n = W // blocks
+    lengths, cuts = [203, 141], [[130, 1, 2, 64, 5, 1], [1, 70, 2, 65, 2, 1]]
+    full = [torch.randn(L, 2 * W + 8, generator=g).to(dtype) for L in lengths]
+    cw, cb = 0.6 * torch.randn(W, taps, generator=g), 0.3 * torch.randn(W, generator=g)
+    gw = (torch.randn(2, blocks, n, n, generator=g) / n ** 0.5).to(dtype)
+    gb = 0.3 * torch.randn(2, W, generator=g)
+    lam = torch.linspace(-9.0, 1.0, W)
+    tails = torch.zeros(4, taps - 1, W, device=device)
+    state = torch.zeros(4, W, device=device)
+    slots, got, at = ints([2, 0], device), [[], []], [0, 0]
+    for s in range(6):
+        m, cu, seq, tiles, tc, _ = layout(lengths, cuts, s, device)
+        proj = torch.cat([full[b][at[b]:at[b] + m[b]] for b in (0, 1)]).to(device)[:, :2 * W]
+        o = SM.linear_unit(proj, cw.to(device), cb.to(device), tails, gw.to(device), gb.to(device),
+                           lam.to(device), 8.0, state, cu, seq, slots, dtype, tiles, tc)
+        got[0].append(o[:m[0]])
+        got[1].append(o[m[0]:])
+        at = [a + k for a, k in zip(at, m)]
+    for b in (0, 1):
+        x = full[b][:, :2 * W].double()
+        u = O.short_conv(x[:, W:], cw.double(), cb.double())
+        r, i = (torch.sigmoid(O.block_linear(gw[k].double(), gb[k].double().view(blocks, n), u))
+                for k in (0, 1))
+        S = O.linear_unit(u, r, i, lam.double())
+        want = S * O.gelu_tanh(x[:, :W])
+        assert rel_err(torch.cat(got[b]).float(), want) < (1e-5 if dtype == torch.float32 else 5e-3)
+        assert rel_err(state[2 - 2 * b], S[-1]) < (1e-5 if dtype == torch.float32 else 1e-4)
+        for k in range(taps - 1):
+            assert rel_err(tails[2 - 2 * b, k], x[lengths[b] - taps + 1 + k, W:]) < 1e-6
+
+
+@pytest.mark.parametrize("E,top,groups", [(12, 4, (4, 3)), (6, 2, (3, 1)), (6, 3, (2, 1)),
+                                          (5, 3, None), (8, 8, (4, 4)), (9, 2, (9, 2)), (1, 1, None),
+                                          (64, 6, (8, 3))])
+def test_router_and_experts(dev, E, top, groups):
+    device, dtype = dev
+    g = torch.Generator().manual_seed(E)
+    T, D, ff = 37, 24, 10
+    h = torch.randn(T, D, generator=g).to(dtype)
+    rw = 2.0 * torch.randn(E, D, generator=g)
+    idx, wts = SM.moe_route_all(h.to(device), rw.to(device), None, top, 1.0, groups, True)
+    rc = {"top": top}
+    if groups:
+        rc["groups"] = {"count": groups[0], "keep": groups[1]}
+    z = h.double() @ rw.double().t()
+    for t in range(T):
+        want = O.choose(z[t], rc)
+        assert idx[t].tolist() == [e for e, _ in want]
+        assert wts[t].tolist() == pytest.approx([v for _, v in want], rel=1e-4, abs=1e-7)
+    # weights are scores over their sum, whatever the scale
+    _, twice = SM.moe_route_all(h.to(device), rw.to(device), None, top, 2.0, groups, True)
+    assert rel_err(twice, 2.0 * wts) < 1e-6
+    up = (torch.randn(E, ff, D, generator=g) / D ** 0.5).to(dtype)
+    down = (torch.randn(E, D, ff, generator=g) / ff ** 0.5).to(dtype)
+    for rows in (T, 2):                             # prompt and decode forms
+        got = SM.moe_experts_relu2(h[:rows].to(device), idx[:rows], wts[:rows], up.to(device),
+                                   down.to(device))
+        w = {}
+        for e in range(E):
+            w[f"e{e}.up"], w[f"e{e}.down"] = up[e], down[e]
+        want = torch.zeros(rows, D, dtype=torch.float64)
+        for t in range(rows):
+            for e, v in O.choose(z[t], rc):
+                a = torch.relu(O._lin(w, f"e{e}.up", h[t].double())) ** 2
+                want[t] += v * O._lin(w, f"e{e}.down", a)
+        assert rel_err(got, want) < (1e-5 if dtype == torch.float32 else 8e-3)
+
+
+def test_best_group_rule(dev):
+    """A group counts by its best member: the second best expert overall is
+    out of reach when it shares no kept group, however good the rest is."""
+    device, _ = dev
+    rw = torch.tensor([[9.0], [0.0], [8.0], [7.9], [8.5], [-5.0]])
+    h = torch.ones(1, 1)
+    idx, _ = SM.moe_route_all(h.to(device), rw.to(device), None, 2, 1.0, (3, 1), True)
+    assert idx[0].tolist() == [0, 1]
+    idx, _ = SM.moe_route_all(h.to(device), rw.to(device), None, 3, 1.0, (3, 2), True)
+    assert idx[0].tolist() == [0, 4, 1]
+    idx, _ = SM.moe_route_all(h.to(device), rw.to(device), None, 3, 1.0, (3, 3), True)
+    assert idx[0].tolist() == [0, 4, 2]
+
+
+@pytest.mark.parametrize("H,G,dk,dv,rot_dims", [(4, 2, 8, 5, 6), (3, 3, 6, 4, 0), (2, 1, 72, 4, 72)])
+def test_prepare(dev, H, G, dk, dv, rot_dims):
+    """Weighted q/k norm, then half rotary, then the page write."""
+    device, dtype = dev
+    g = torch.Generator().manual_seed(2)
+    T, eps = 9, 1e-3
+    n = (H + G) * dk + G * dv
+    x = torch.randn(T, n + 6, generator=g).to(dtype)
+    qw, kw = (1.0 + 0.3 * torch.randn(dk, generator=g) for _ in range(2))
+    pos = [0, 1, 5, 63, 64, 500, 1000, 4000, 2]
+    page = [3, 17, 0, 8, 5, 11, 2, 19, 9]
+    freqs = None
+    if rot_dims:
+        freqs = torch.tensor(rotary_frequencies(rot_dims, 70.0)[0],
+                             dtype=torch.float64).float().to(device)
+    cache = torch.zeros(20, G * (dk + dv), dtype=dtype, device=device)
+    q = SM.qk_prepare_kv_write(x.to(device)[:, :n], H, G, dk, dv, qw.to(device), kw.to(device), eps,
+                               ints(pos, device), freqs, 1.0, None, ints(page, device), cache)
+    rot = {"base": 70.0, "dims": rot_dims}
+    xd = x.double()
+    wq = O.rms_unit(xd[:, :H * dk].reshape(T, H, dk), eps) * qw.double()
+    wk = O.rms_unit(xd[:, H * dk:(H + G) * dk].reshape(T, G, dk), eps) * kw.double()
+    wq = torch.stack([O.rotate_halves(wq[t], pos[t], rot) for t in range(T)])
+    wk = torch.stack([O.rotate_halves(wk[t], pos[t], rot) for t in range(T)])
+    bound = 2e-4 if dtype == torch.float32 else 6e-3        # fp32 angles at position 4000
+    assert rel_err(q.float(), wq) < bound
+    want = torch.cat([wk.reshape(T, -1), xd[:, (H + G) * dk:n]], -1)
+    assert rel_err(cache[torch.tensor(page).to(device)].float(), want) < bound
+
+
+def _paged(device, dtype, width, bs, lengths, seed):
+    """Random cache rows for sequences of the given lengths, in pages of
+    random order: (cache, block tables, rows per sequence)."""
+    g = torch.Generator().manual_seed(seed)
+    nblk = sum((n + bs - 1) // bs for n in lengths)
+    perm = torch.randperm(nblk, generator=g).tolist()
+    cache = torch.zeros((nblk + 1) * bs, width, dtype=dtype, device=device)
+    tables, kv = [], []
+    for n in lengths:
+        tables.append([perm.pop() for _ in range((n + bs - 1) // bs)])
+        kv.append(torch.randn(n, width, generator=g).to(dtype).float())
+    most = max(len(t) for t in tables)
+    return cache, [t + [0] * (most - len(t)) for t in tables], kv
+
+
+def _attention(device, dtype, H, G, dk, dv, chunk, softcap, sinks, bs, lengths, news, seed=0,
+               tweak=None, window=0, keep=0):
+    """-> (kernel result, direct float64 result) for the last ``news`` tokens
+    of every sequence. ``tweak(kv, q)`` may change rows and queries first."""
+    W = G * (dk + dv)
+    cache, tables, kv = _paged(device, dtype, W, bs, lengths, seed)
+    g = torch.Generator().manual_seed(seed + 50)
+    T = sum(news)
+    q = (2.0 * torch.randn(T, H, dk, generator=g)).to(dtype)
+    sink = torch.randn(H, generator=g) + 1.0 if sinks is True else sinks
+    if tweak is not None:
+        tweak(kv, q)
+    kv = [r.to(dtype) for r in kv]
+    for b, rows in enumerate(kv):
+        idx = torch.tensor([tables[b][j // bs] * bs + j % bs for j in range(lengths[b])])
+        cache[idx.to(device)] = rows.to(device)
+    pos, seq, cu = [], [], [0]
+    for b, (n, m) in enumerate(zip(lengths, news)):
+        pos += list(range(n - m, n))
+        seq += [b] * m
+        cu.append(cu[-1] + m)
+    tiles, mt = SM.query_tiles(news, SM.WIDE_QUERY_TILE)
+    got = SM.window_attention(
+        q.to(device), cache, H, G, dk, dv, False, ints(tables, device), bs, ints(cu, device),
+        ints(seq, device), ints(pos, device), 0.31, window, keep, None, None, None, dtype,
+        tiles=ints(tiles, device), max_tile=mt, chunk=chunk, softcap=softcap,
+        sink=None if sink is None else sink.to(device))
+    want = torch.zeros(T, H, dv, dtype=torch.float64)
+    for t in range(T):
+        rows, p = kv[seq[t]].double(), pos[t]
+        lo = max(O.first_visible(p, {"size": chunk}), p - window + 1 if window else 0)
+        see = [j for j in range(p + 1) if j >= lo or j < keep]
+        for a in range(H):
+            c = a // (H // G)
+            s = rows[see, c * dk:(c + 1) * dk] @ q[t, a].double() * 0.31
+            s = O.capped(s, softcap)
+            wt = torch.softmax(s, -1) if sink is None else O.sink_softmax(s, sink[a])
+            want[t, a] = wt @ rows[see, G * dk + c * dv:G * dk + (c + 1) * dv]
+    return got, want.reshape(T, H * dv)
+
+
+@pytest.mark.parametrize("H,G,dk,dv,chunk,softcap,sinks", [
+    (4, 2, 6, 10, 7, 2.0, True), (3, 1, 8, 8, 16, 0.0, True), (6, 2, 8, 6, 5, 3.0, None),
+    (2, 2, 8, 6, 0, 1.5, True), (5, 1, 7, 3, 4, 2.0, True), (3, 3, 8, 1, 1, 2.0, True)])
+def test_attention_op(dev, H, G, dk, dv, chunk, softcap, sinks):
+    """Prompt portions and single tokens in one step against direct softmaxes:
+    chunks, caps, sinks, pages in random order."""
+    got, want = _attention(*dev, H, G, dk, dv, chunk, softcap, sinks, 4, [23, 9, 14, 1],
+                           [11, 1, 14, 1])
+    assert rel_err(got.float(), want) < (1e-5 if dev[1] == torch.float32 else 1e-2)
+
+
+@pytest.mark.parametrize("window,keep,chunk", [(6, 0, 9), (20, 3, 8), (5, 2, 0), (0, 4, 7)])
+def test_chunks_beside_windows_and_kept_tokens(dev, window, keep, chunk):
+    """The visibility rules combine: the later start of window and chunk, and
+    kept first tokens with either."""
+    got, want = _attention(*dev, 4, 2, 8, 8, chunk, 2.0, True, 4, [41, 9, 30], [30, 1, 1],
+                           window=window, keep=keep)
+    assert rel_err(got.float(), want) < (1e-5 if dev[1] == torch.float32 else 1e-2)
+
+
+@pytest.mark.parametrize("m", [1, 3, 9])
+def test_chunk_edges_of_the_op(dev, m):
+    """A key that stands out counts at the first place of the query's chunk and
+    not one place before; at page borders; from a decoded token and portions
+    that lie inside a chunk or cross its border."""
+    H, G, dk, dv, chunk = 2, 1, 8, 8, 12
+    for n in (60, 61, 67, 72, 73):
+        edge = (n - 1) // chunk * chunk
+        for j_star in {edge, edge - 1, n - 1, 0, 15, 16}:
+            seen = edge <= j_star <= n - 1
+
+            def tweak(kv, q):
+                kv[0] *= 0.05
+                kv[0][j_star, :dk] = 4.0
+                kv[0][j_star, dk:] = torch.arange(1, dv + 1).float()
+                q[:] = 4.0
+            got, want = _attention(*dev, H, G, dk, dv, chunk, 30.0, torch.tensor([-2.0, -1.0]), 4,
+                                   [n], [m], tweak=tweak)
+            assert rel_err(got.float(), want) < (1e-5 if dev[1] == torch.float32 else 2e-2)
+            last = got[-1].float().cpu().view(H, dv)
+            if seen:
+                assert rel_err(last[0], torch.arange(1, dv + 1).double()) < 2e-2, (n, j_star)
+            else:
+                assert float(last.abs().max()) < 0.2, (n, j_star)
+
+
+@pytest.mark.parametrize("m", [1, 3, 9])
+def test_sink_and_cap_of_the_op(dev, m):
+    """The sink counts once, is not scaled and not capped, and holds its own
+    value: with all scores equal to s the weights are e^s / (k e^s + e^sink)."""
+    device, dtype = dev
+    H, G, dk, dv, n, cap = 2, 2, 8, 4, 300, 2.0
+
+    def tweak(kv, q):
+        kv[0][:, :G * dk] = 1.0
+        kv[0][:, G * dk:] = 1.0
+        q[:] = 1.0
+    sink = torch.tensor([6.0, -30.0])
+    got, want = _attention(device, dtype, H, G, dk, dv, 0, cap, sink, 16, [n], [m], tweak=tweak)
+    s = cap * torch.tanh(torch.tensor(8 * 0.31 / cap, dtype=torch.float64))
+    flat = got[-1].double().cpu().view(H, dv)
+    bound = 1e-5 if dtype == torch.float32 else 5e-3
+    share = float(n * s.exp() / (n * s.exp() + sink[0].double().exp()))
+    assert rel_err(flat[0], torch.full((dv,), share)) < bound
+    assert rel_err(flat[1], torch.ones(dv)) < bound
+    assert rel_err(got.float(), want) < bound
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("H,G,dk,dv,chunk,softcap,sinks,lengths,news", [
+    (4, 2, 64, 128, 100, 20.0, True, [300, 70, 129], [200, 70, 65]),
+    (8, 2, 40, 80, 77, 4.0, True, [257, 64], [257, 5]),
+    (2, 2, 128, 256, 33, 0.0, True, [190], [140]),
+    (3, 1, 72, 64, 64, 3.0, None, [333, 21], [333, 21]),
+    (2, 1, 200, 40, 150, 5.0, True, [257], [257]),
+    (2, 1, 16, 8, 0, 5.0, True, [257], [100]),
+])
+def test_tiled_attention_kernel(H, G, dk, dv, chunk, softcap, sinks, lengths, news):
+    """The bf16 MFMA kernel against float64: chunk borders inside and between
+    query tiles and key blocks, caps and sinks at every register variant."""
+    got, want = _attention("cuda", torch.bfloat16, H, G, dk, dv, chunk, softcap, sinks, 16, lengths,
+                           news, seed=7)
+    assert rel_err(got.float(), want) < 1e-2
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("H,G,dk,dv,chunk,lengths", [
+    (8, 2, 64, 128, 0, [700, 40, 1, 333]), (4, 4, 32, 16, 1000, [1500, 9]),
+    (6, 1, 16, 24, 64, [64, 65, 63, 200]), (8, 1, 8, 250, 333, [700, 90]),
+    (3, 1, 40, 8, 128, [129, 135, 600])])
+def test_grouped_attention_kernel(dtype, H, G, dk, dv, chunk, lengths):
+    """Decode steps through the grouped kernel and its merge of key shares:
+    the sink joins once however the keys are shared out."""
+    got, want = _attention("cuda", dtype, H, G, dk, dv, chunk, 4.0, True, 16, lengths,
+                           [1] * len(lengths), seed=9)
+    assert rel_err(got.float(), want) < (1e-5 if dtype == torch.float32 else 1e-2)
+
+
+# ------------------------------------------------------------ whole models
+
+@pytest.mark.parametrize("which", ["lightning", "pair", "dense", "moe"])
+def test_single_layer_models(dev, which):
+    layer = {"lightning": O.light_layer(), "pair": O.pair_layer(),
+             "dense": O.light_layer(mlp=O.dense()), "moe": O.pair_layer(mlp=O.moe())}[which]
+    cfg = O.make_cfg([layer], width=24, vocab=31)
+    W, eng = build(cfg, dev)
+    t = toks(25, 31, seed=3)
+    want = O.forward(cfg, W, t)
+    assert rel_err(run_portions(eng, t, [25]), want) < tol(dev[1])
+    assert rel_err(run_portions(eng, t, [9] + [1] * 16), want) < tol(dev[1])
+
+
+@pytest.mark.parametrize("make,n", [(mixed_cfg, 45), (aligned_cfg, 150)])
+def test_whole_prompt_and_layers(dev, make, n):
+    cfg = make()
+    W, eng = build(cfg, dev)
+    t = toks(n, cfg["vocab"], seed=4)
+    lay, cap = [], []
+    want = O.forward(cfg, W, t, lay)
+    got = run_portions(eng, t, [n], capture=cap)
+    assert len(cap) == len(lay) == len(eng.spec.runs)    # a looped layer counts each time
+    for i, (a, b) in enumerate(zip(cap, lay)):
+        assert rel_err(a, b) < tol(dev[1]), i
+    assert rel_err(got, want) < tol(dev[1])
+    # without the capture the pass injection is fused into the layer tail
+    assert rel_err(run_portions(eng, t, [n]), want) < tol(dev[1])
+
+
+@pytest.mark.parametrize("loop", [None, (0, 1, 3), (1, 2, 3), (0, 2, 2), (1, 1, 4), (0, 2, 1),
+                                  (1, 2, 1)])
+def test_loops(dev, loop):
+    """Stretches of one and two layers at the start, at the end and over the
+    whole model; a single pass gets its vector; an empty stretch adds nothing."""
+    cfg = O.make_cfg([O.light_layer(mlp=O.dense(8)), O.pair_layer()], width=16, vocab=31, loop=loop)
+    W, eng = build(cfg, dev)
+    runs = O.layer_runs(cfg)
+    assert eng.spec.pass_starts == {r: t for r, (_, t) in enumerate(runs) if t is not None}
+    assert len(eng.slots.recurrent) == len(runs)
+    t = toks(23, 31, seed=8)
+    want = O.forward(cfg, W, t)
+    assert rel_err(run_portions(eng, t, [23]), want) < tol(dev[1])
+    assert rel_err(run_portions(eng, t, [3, 2, 9] + [1] * 9), want) < tol(dev[1])
+
+
+def test_first_tokens(dev):
+    """Sequences of one to five tokens, alone and token by token."""
+    cfg = mixed_cfg()
+    W, eng = build(cfg, dev)
+    for n in (1, 2, 3, 4, 5):
+        t = toks(n, 37, seed=5 + n)
+        want = O.forward(cfg, W, t)
+        assert rel_err(run_portions(eng, t, [n]), want) < tol(dev[1])
+        assert rel_err(run_portions(eng, t, [1] * n), want) < tol(dev[1])
+
+
+@pytest.mark.parametrize("cuts", [[1] * 30, [2] * 15, [7, 2, 2, 1, 11, 3, 4], [16, 14], [29, 1],
+                                  [3, 27], [15, 2, 13], [5, 25]])
+def test_portions(dev, cuts):
+    cfg = mixed_cfg()
+    W, eng = build(cfg, dev)
+    t = toks(30, 37, seed=6)
+    assert rel_err(run_portions(eng, t, cuts), O.forward(cfg, W, t)) < tol(dev[1])
+
+
+@pytest.mark.parametrize("cuts", [[64, 86], [63, 2, 85], [65, 64, 21], [100, 49, 1], [2] * 75])
+def test_portions_around_tiles(dev, cuts):
+    cfg = aligned_cfg()
+    W, eng = build(cfg, dev)
+    t = toks(150, 41, seed=6)
+    assert rel_err(run_portions(eng, t, cuts), O.forward(cfg, W, t)) < tol(dev[1])
+
+
+def test_portions_do_not_change_fp32_results(dev):
+    if dev[1] != torch.float32:
+        pytest.skip("fp32 statement")
+    cfg = mixed_cfg()
+    W, eng = build(cfg, dev)
+    t = toks(40, 37, seed=7)
+    whole = run_portions(eng, t, [40])
+    for cuts in ([1] * 40, [2] * 20, [13, 5, 2, 20], [39, 1]):
+        assert rel_err(run_portions(eng, t, cuts), whole) < 2e-5
+
+
+@pytest.mark.parametrize("make,big", [(mixed_cfg, 1), (aligned_cfg, 4)])
+def test_mixed_batches_and_reuse(dev, make, big):
+    """Unequal requests in one step (portions beside single tokens, requests
+    sitting steps out), pages and slots given back and taken again; every
+    position against the oracle and against the request run alone."""
+    cfg = make()
+    W, eng = build(cfg, dev, blocks=40 * big, slots=3)
+    V = cfg["vocab"]
+    reqs = {k: toks(n, V, seed=10 + i) for i, (k, n) in
+            enumerate((("a", 26), ("b", 9), ("c", 17), ("d", 22), ("e", 5)))}
+    plan = [[("a", 7), ("b", 2)], [("a", 1), ("b", 3), ("c", 9)], [("a", 1), ("c", 2)],
+            [("a", 6), ("b", 4), ("c", 1)], [("c", 5), ("a", 1)], [("a", 10), ("d", 3)],
+            [("d", 1), ("e", 2)], [("d", 12), ("e", 1)], [("d", 6), ("e", 2)]]
+    if big > 1:                                     # portions over tile borders
+        plan = [[(k, n if n == 1 else n * big) for k, n in s] for s in plan]
+        reqs = {k: toks(sum(n for s in plan for kk, n in s if kk == k), V, seed=10 + i)
+                for i, k in enumerate(reqs)}
+    live, at, got = {}, {k: 0 for k in reqs}, {k: [] for k in reqs}
+    for stepn in plan:
+        work, want = [], []
+        for k, n in stepn:
+            if k not in live:
+                live[k] = eng.open_sequence()
+            work.append((live[k], reqs[k][at[k]:at[k] + n]))
+            want.append(list(range(n)))
+        out = eng.step(work, want)
+        o = 0
+        for k, n in stepn:
+            got[k].append(out[o:o + n])
+            o += n
+            at[k] += n
+            if at[k] == len(reqs[k]):
+                eng.close_sequence(live.pop(k))
+    assert not live
+    _, solo = build(cfg, dev, W=W)
+    for k, t in reqs.items():
+        g = torch.cat(got[k])
+        assert rel_err(g, O.forward(cfg, W, t)) < tol(dev[1]), k
+        alone = run_portions(solo, t, [len(t)])
+        assert rel_err(g, alone) < (1e-5 if dev[1] == torch.float32 else 0.06), k
+
+
+def test_dirty_pages_and_slots(dev):
+    """Freed pages, states and convolution tails hold another request's
+    leftovers."""
+    cfg = mixed_cfg()
+    W, eng = build(cfg, dev, blocks=12, slots=1)
+    a, b = toks(40, 37, seed=20), toks(35, 37, seed=21)
+    run_portions(eng, a, [40])
+    for r in (list(eng.pool.rows.values()) + list(eng.slots.recurrent.values())
+              + list(eng.slots.mixer_tails.values())):
+        r.add_(5.0)
+    assert rel_err(run_portions(eng, b, [20, 15]), O.forward(cfg, W, b)) < tol(dev[1])
+    assert eng.pool.allocator.num_free == 12 and eng.slots.num_free == 1
+
+
+def test_long_decode(dev):
+    """120 single-token steps: many chunk borders pass, the states carry on."""
+    cfg = O.make_cfg([O.light_layer(mlp=O.moe()), O.pair_layer(chunk=9)], width=16, vocab=31,
+                     loop=(0, 2, 2))
+    W, eng = build(cfg, dev, blocks=48)
+    t = toks(132, 31, seed=30)
+    got = run_portions(eng, t, [12] + [1] * 120)
+    want = O.forward(cfg, W, t)
+    assert rel_err(got, want) < tol(dev[1])
+    assert rel_err(got[-20:], want[-20:]) < tol(dev[1])
+
+
+@pytest.mark.parametrize("which", ["lightning", "unit"])
+def test_state_reaches_far_back(dev, which):
+    """With slow decays and a few loud tokens 230 places back, the last logits
+    depend on it through the state alone, from portions and decoded; with fast
+    decays they do not."""
+    device, dtype = dev
+    for slow in (True, False):
+        if which == "lightning":
+            layer = O.light_layer(heads=2, decay=[0.9999, 0.9995] if slow else [0.3, 0.5])
+        else:
+            layer = O.pair_layer(chunk=8, width=16, blocks=2)
+        cfg = O.make_cfg([layer], width=16, vocab=31, embed_scale=0.5)
+        W = O.random_weights(cfg, 6)
+        if which == "unit":
+            W["l0.mix.right.lam"] = torch.full((16,), -8.0 if slow else 1.0)
+            W["l0.mix.left.out"] = torch.zeros(16)
+        # token 30's row points one way and nothing else does
+        W["embed"][:, 0] = 0.0
+        W["embed"][30] = 0.0
+        W["embed"][30, 0] = 8.0
+        for n in ("l0.mix.k", "l0.mix.v") if which == "lightning" else ("l0.mix.right.x",):
+            W[n][:, 0] = 6.0
+        W = {k: v.to(torch.bfloat16).float() for k, v in W.items()}
+        W, eng = build(cfg, dev, blocks=96, W=W)
+        base = [x % 30 for x in toks(250, 31, seed=41)]
+        alt = list(base)
+        alt[14:20] = [30] * 6
+        far = [O.forward(cfg, W, t)[-1] for t in (base, alt)]
+        moved = rel_err(far[1], far[0])
+        assert (moved > 0.05) if slow else (moved < 1e-3), moved
+        for t, want in zip((base, alt), far):
+            for cuts in ([250], [130, 115] + [1] * 5):
+                assert rel_err(run_portions(eng, t, cuts)[-1], want) < (
+                    2e-4 if dtype == torch.float32 else 0.05)
+
+
+def test_chunk_edges_in_model(dev):
+    """With the recurrent side silenced, moving the first token of the chunk
+    changes a later position's logits and the one before it does not."""
+    device, dtype = dev
+    cfg = O.make_cfg([O.pair_layer(chunk=6)], width=16, vocab=31)
+    W = O.random_weights(cfg, 2)
+    W["l0.mix.right.out"] = torch.zeros_like(W["l0.mix.right.out"])
+    W, eng = build(cfg, dev, W=W)
+    for n in (18, 20, 23, 24):                      # the last token at four places of its chunk
+        base = toks(n, 31, seed=40)
+        ref = run_portions(eng, base, [10] + [1] * (n - 10))[-1]
+        edge = (n - 1) // 6 * 6
+        for j, seen in ((edge, True), (edge - 1, False), (0, False)):
+            alt = list(base)
+            alt[j] = (alt[j] + 7) % 31
+            for cuts in ([n], [10] + [1] * (n - 10), [13, 2, n - 15]):
+                out = run_portions(eng, alt, cuts)[-1]
+                moved = rel_err(out, ref)
+                # between two ways of cutting, bf16 rounding moves logits a little
+                floor = 1e-3 if dtype == torch.float32 else 2e-2
+                assert (moved > floor) == seen, (n, j, cuts, moved)
+                assert rel_err(out, O.forward(cfg, W, alt)[-1]) < tol(dtype)
+
+
+def test_sinks_in_model(dev):
+    """A large sink silences its head: the oracle with the sinks left out is
+    far from the model."""
+    cfg = O.make_cfg([O.pair_layer(chunk=9)], width=16, vocab=31)
+    W = O.random_weights(cfg, 3)
+    W["l0.mix.left.sink"] = torch.tensor([4.0, -3.0, 2.0, 5.0])
+    W, eng = build(cfg, dev, W=W)
+    t = toks(20, 31, seed=44)
+    want = O.forward(cfg, W, t)
+    for cuts in ([20], [7] + [1] * 13):
+        assert rel_err(run_portions(eng, t, cuts), want) < tol(dev[1])
+    none = dict(W)
+    none["l0.mix.left.sink"] = torch.full((4,), -100.0)
+    assert rel_err(O.forward(cfg, none, t), want) > 0.15
+
+
+def test_other_sizes(dev):
+    """Values a model may happen to make equal or 1: one head, chunks of one
+    token, one tap, one block and a block per channel, rotation over the whole
+    head and none, unit scales, one expert, every group kept, no cap."""
+    cfg = O.make_cfg([
+        O.light_layer(heads=1, dim=8, vdim=8, decay=[1.0], mlp=O.moe(1, 1, 8, (1, 1))),
+        O.pair_layer(heads=1, kv_heads=1, dim=8, vdim=8, chunk=1, rot_dims=8, scale=1.0,
+                     softcap=0.0, width=8, blocks=8, conv=1, mlp=O.dense(8)),
+        O.light_layer(heads=8, dim=1, vdim=1, mlp=O.moe(8, 8, 8, (8, 8))),
+        O.pair_layer(heads=8, kv_heads=1, dim=8, vdim=8, chunk=8, rot_dims=0, width=8, blocks=1,
+                     conv=8, mlp=O.moe(8, 1, 8, (8, 1))),
+    ], width=8, vocab=11, embed_scale=1.0)
+    W, eng = build(cfg, dev)
+    t = toks(21, 11, seed=50)
+    want = O.forward(cfg, W, t)
+    assert rel_err(run_portions(eng, t, [21]), want) < tol(dev[1])
+    assert rel_err(run_portions(eng, t, [5, 2, 1, 13]), want) < tol(dev[1])
+    no_mask = O.pair_layer(heads=5, kv_heads=1, dim=10, vdim=14, width=30, blocks=5, conv=6,
+                           mlp=O.dense(9))
+    for k in ("mask", "softcap", "rot"):            # absent: full causal, plain scores
+        del no_mask["mixer"]["left"][k]
+    cfg = O.make_cfg([O.light_layer(heads=5, dim=3, vdim=7, mlp=O.moe(10, 4, 6, (5, 3))), no_mask],
+                     width=30, vocab=19, loop=(0, 1, 4))
+    W, eng = build(cfg, dev)
+    t = toks(19, 19, seed=51)
+    assert rel_err(run_portions(eng, t, [6, 13]), O.forward(cfg, W, t)) < tol(dev[1])
+    assert rel_err(run_portions(eng, t, [6] + [1] * 13), O.forward(cfg, W, t)) < tol(dev[1])
+
+
+def test_greedy_generate(dev):
+    """Greedy decoding through generate() and its scheduler (small step
+    budget, two prompts): every generated token is the oracle's argmax for
+    its prefix wherever the oracle's margin is not a rounding matter."""
+    cfg = mixed_cfg()
+    W, eng = build(cfg, dev, blocks=64, slots=4)
+    eng.cfg.step_token_budget = 8
+    prompts = [toks(13, 37, seed=60), toks(6, 37, seed=61)]
+    outs = eng.generate(prompts, SamplingParams(max_tokens=10, temperature=0.0, n=1))
+    checked = 0
+    for p, o in zip(prompts, outs):
+        gen = o[0]
+        assert len(gen) == 10
+        logits = O.forward(cfg, W, p + gen)
+        margin = (1e-3 if dev[1] == torch.float32 else 0.3) * float(logits.std())
+        for i, tok in enumerate(gen):
+            row = logits[len(p) - 1 + i]
+            top2 = torch.topk(row, 2).values
+            if float(top2[0] - top2[1]) > margin:
+                assert int(row.argmax()) == tok, (i, tok)
+                checked += 1
+    assert checked >= 5
+    assert eng.slots.num_free == 4 and eng.pool.allocator.num_free == 64
+
+
+def test_fork_shares_pages_and_copies_state(dev):
+    cfg = mixed_cfg()
+    W, eng = build(cfg, dev, blocks=20, block_size=4)
+    t = toks(18, 37, seed=33)
+    q = eng.open_sequence()
+    eng.step([(q, t[:10])], [[]])
+    c = eng.fork_sequence(q)
+    tail2 = [(x + 3) % 37 for x in t[10:]]
+    out = eng.step([(q, t[10:]), (c, tail2)], [list(range(8)), list(range(8))])
+    assert rel_err(out[:8], O.forward(cfg, W, t)[10:]) < tol(dev[1])
+    assert rel_err(out[8:], O.forward(cfg, W, t[:10] + tail2)[10:]) < tol(dev[1])
+    eng.close_sequence(q)
+    eng.close_sequence(c)
+    assert eng.pool.allocator.num_free == 20
+
+
+def test_served_through_the_batcher():
+    """The server's app, batcher and sampler drive the design's engine like
+    any other: greedy completions repeat, sampled ones fan out."""
+    from fastapi.testclient import TestClient
+
+    from distrl_llm_amd.serve import create_app
+    from distrl_llm_amd.utils.tokenizer import ByteTokenizer
+    cfg = O.make_cfg([O.light_layer(mlp=O.dense(8)), O.pair_layer(mlp=O.moe())], width=16,
+                     vocab=600, loop=(0, 1, 2))
+    _, eng = build(cfg, ("cpu", torch.float32), blocks=128, block_size=8, slots=8)
+    client = TestClient(create_app(eng, ByteTokenizer(vocab_size=600), "tiny-pedazen"))
+    body = {"prompt": "2+2=", "max_tokens": 5, "temperature": 0.0}
+    a = client.post("/v1/completions", json=body).json()
+    b = client.post("/v1/completions", json=body).json()
+    assert a["choices"][0]["text"] == b["choices"][0]["text"]
+    assert a["usage"]["completion_tokens"] <= 5
+    r = client.post("/v1/completions", json={"prompt": ["abcd", "wxyz"], "max_tokens": 3,
+                                             "temperature": 1.0, "top_p": 0.9, "n": 2}).json()
+    assert len(r["choices"]) == 4
+    assert eng.pool.allocator.num_free == 128 and eng.slots.num_free == 8
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("make", [mixed_cfg, aligned_cfg])
+def test_captured_decode_matches_eager(dtype, make):
+    """Every replay of the captured step against the eager step, with eager
+    work (another sequence's portion) between the replays."""
+    cfg = make()
+    V = cfg["vocab"]
+    dev = ("cuda", dtype)
+    W, eng = build(cfg, dev)
+    _, eager = build(cfg, dev, W=W)
+    eager.cfg.enforce_eager = True
+    t, other = toks(30, V, seed=70), toks(20, V, seed=71)
+    qa, qb, qc = eng.open_sequence(), eager.open_sequence(), eng.open_sequence()
+    for q, e in ((qa, eng), (qb, eager)):
+        e.step([(q, t[:10])], [[9]])
+    for i in range(10, 30):
+        a = eng.step([(qa, t[i:i + 1])])
+        b = eager.step([(qb, t[i:i + 1])])
+        assert rel_err(a, b) < 1e-5, i
+        if i % 4 == 0:
+            eng.step([(qc, other[i - 10:i - 8])], [[1]])
+            torch.cuda.synchronize()
+    assert len(eng._decode_graphs) >= 1
+
+
+# --------------------------------------------------- files, registry, tools
+
+def test_checkpoint_registry_and_replay(tmp_path):
+    """Save a checkpoint, load it through the registry, replay a step trace
+    with the command-line tool and compare with the oracle."""
+    from distrl_llm_amd.models.registry import hybrid_design_of, load_model_and_engine
+    cfg = mixed_cfg()
+    W = O.random_weights(cfg, 3)
+    model = HybridLM(pedazen_spec_from_config(cfg), dtype=torch.float32, device="cpu")
+    model.load_tensors(W)
+    assert pedazen_spec_from_config(pedazen_config_from_spec(model.spec),
+                                    model.spec.name) == model.spec
+    path = str(tmp_path / "tiny")
+    save_pedazen_checkpoint(model, path)
+    assert hybrid_design_of(path) == "pedazen"
+    m2, eng = load_model_and_engine(path, EngineConfig(max_seq_length=256, kv_block_size=4,
+                                                       num_kv_blocks=32, num_state_slots=2,
+                                                       max_num_seqs=2),
+                                    dtype=torch.float32, device=torch.device("cpu"))
+    again = m2.export_tensors()
+    for k, v in model.export_tensors().items():
+        assert torch.equal(v, again[k]) and v.shape == W[k].shape, k
+        assert torch.equal(v.float(), W[k]), k
+    a, b = toks(21, 37, seed=80), toks(11, 37, seed=81)
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:9], "want": [8]},
+                                     {"id": "b", "tokens": b[:2], "want": []}], "end": []},
+             {"step": 1, "entries": [{"id": "b", "tokens": b[2:], "want": [0, 8]},
+                                     {"id": "a", "tokens": a[9:10], "want": [0]}], "end": ["b"]},
+             {"step": 2, "entries": [{"id": "a", "tokens": a[10:], "want": [10]}], "end": ["a"]}]
+    out = tmp_path / "out"
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    env = dict(os.environ, CUDA_VISIBLE_DEVICES="", HIP_VISIBLE_DEVICES="")
+    r = subprocess.run([sys.executable, os.path.join(root, "bin", "trace_run"), "--model", path,
+                        "--dtype", "float32", "--out", str(out), "--max-tokens", "64"],
+                       input="\n".join(json.dumps(s) for s in steps) + "\n", text=True,
+                       capture_output=True, env=env, timeout=300)
+    assert r.returncode == 0, r.stderr[-2000:]
+    assert [ln for ln in r.stdout.split("\n") if ln.startswith("done")] == [
+        "done 0", "done 1", "done 2"]
+    import numpy as np
+    la, lb = O.forward(cfg, W, a), O.forward(cfg, W, b)
+    want = {0: la[8:9], 1: torch.stack([lb[2], lb[10], la[9]]), 2: la[20:21]}
+    for n, w in want.items():
+        got = torch.from_numpy(np.fromfile(out / f"{n}.f32", dtype="<f4").reshape(-1, 37))
+        assert rel_err(got, w) < 2e-4, n
+
+
+def test_loader_names_what_is_missing(tmp_path):
+    from safetensors.torch import load_file, save_file
+    from distrl_llm_amd.models.hybrid import load_pedazen_checkpoint
+    cfg = O.make_cfg([O.pair_layer()], width=16, vocab=31)
+    model = HybridLM(pedazen_spec_from_config(cfg), dtype=torch.float32, device="cpu")
+    model.random_init(1)
+    path = str(tmp_path / "m")
+    save_pedazen_checkpoint(model, path)
+    f = os.path.join(path, "model.safetensors")
+    t = load_file(f)
+    save_file({**t, "extra.table": torch.zeros(2)}, f)       # unnamed tensors are left out
+    load_pedazen_checkpoint(path, dtype=torch.float32)
+    save_file({k: v for k, v in t.items() if k != "l0.mix.right.lam"}, f)
+    with pytest.raises(ValueError, match="right.lam"):
+        load_pedazen_checkpoint(path, dtype=torch.float32)
+
+
+def test_config_errors():
+    good = mixed_cfg()
+    pedazen_spec_from_config(good)
+
+    def broken(change):
+        cfg = json.loads(json.dumps(good))
+        change(cfg)
+        with pytest.raises((ValueError, KeyError)):
+            pedazen_spec_from_config(cfg)
+
+    broken(lambda c: c["layers"][0].update(type="attention"))
+    broken(lambda c: c["layers"][0]["mixer"]["decay"].append(0.5))
+    broken(lambda c: c["layers"][0]["mixer"].pop("vdim"))
+    broken(lambda c: c["layers"][1]["mixer"]["left"].update(kv_heads=4))
+    broken(lambda c: c["layers"][1]["mixer"]["left"]["rot"].update(dims=5))
+    broken(lambda c: c["layers"][1]["mixer"]["left"]["rot"].update(dims=10))
+    broken(lambda c: c["layers"][1]["mixer"]["right"].update(blocks=5))
+    broken(lambda c: c["layers"][1]["mixer"]["right"].update(conv=0))
+    broken(lambda c: c["layers"][1]["mlp"].update(kind="sparse"))
+    broken(lambda c: c["layers"][1]["mlp"]["router"].update(top=7))
+    broken(lambda c: c["layers"][1]["mlp"]["router"]["groups"].update(count=4))
+    broken(lambda c: c["layers"][1]["mlp"]["router"]["groups"].update(keep=4))
+    broken(lambda c: c["layers"][1]["mlp"]["router"].update(top=5))
+    broken(lambda c: c["loop"].update(stop=5))
+    broken(lambda c: c["loop"].update(times=0))

@@ -26,6 +26,10 @@ typedef __attribute__((ext_vector_type(4))) float f32x4;
 namespace {
 
 SM_INLINE float la_silu(float z) { return z * sm_sigmoid(z); }
+SM_INLINE __bf16 la_silu_bf16(__bf16 z) {
+  const float f = (float)z;
+  return (__bf16)(f * sm_fast_sigmoid(f));
+}
 
 // ---- token by token. One workgroup per (row, head, 16 value columns): lane
 // group of 16 per column, a lane holds the keys 64 i + 4 (lane & 15) .. + 3;
@@ -116,7 +120,7 @@ SM_INLINE void la_split(float x, __bf16* hi, __bf16* lo) {
 template <int KS>
 constexpr size_t lac_lds_bytes() {
   return ((size_t)LAC * (KS * 32 + 8) + (size_t)KS * 32 * LAC_TP + 3 * LAC_V * LAC_TP +
-          2 * (size_t)LAC_V * (KS * 32 + 8)) * 2 + 4 * 16 * LAC_PP * 4;
+          2 * (size_t)LAC_V * (KS * 32 + 8)) * 2 + (4 * 16 * LAC_PP + LAC + 4) * 4;
 }
 template <int KS>
 __global__ __launch_bounds__(256, 2) void linear_attention_chunk_kernel(
@@ -133,11 +137,12 @@ __global__ __launch_bounds__(256, 2) void linear_attention_chunk_kernel(
   __bf16* sh = vl + LAC_V * LAC_TP;                       // [LAC_V][KPT] state, hi and lo
   __bf16* sl = sh + LAC_V * KPT;
   float* p_all = reinterpret_cast<float*>(sl + LAC_V * KPT);      // [4][16][LAC_PP]
+  float* pw = p_all + 4 * 16 * LAC_PP;                            // [LAC + 1] powers of the decay
   const int b = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * LAC_V;
   const int tid = threadIdx.x, wave = tid >> 6, l = tid & 63, lrow = l & 15, lk = l >> 4;
   const int t0 = cu[b], n = cu[b + 1] - t0;
   if (n == 0) return;
-  const float* pw = powers + h * np;
+  if (tid <= LAC) pw[tid] = powers[h * np + tid];
   const int nq = H * dk;
   float* st = state + (int64_t)slots[b] * H * vd * dk + (int64_t)h * vd * dk;
   float* p_lds = p_all + wave * 16 * LAC_PP;
@@ -153,46 +158,61 @@ __global__ __launch_bounds__(256, 2) void linear_attention_chunk_kernel(
       if (k < dk && c < vd) sacc[mi][nt] = *reinterpret_cast<const f32x4*>(st + (int64_t)c * dk + k);
     }
 
-  for (int c0 = 0; c0 < n; c0 += LAC) {
+  // a chunk's projection rows, fetched into registers one chunk ahead: the
+  // thread's pieces of k and v, the lane's queries as A fragments
+  constexpr int KI = LAC * (DP / 8) / 256;
+  bf16v8 kraw[KI], vraw, qraw[KS], zero;
+  #pragma unroll
+  for (int j = 0; j < 8; ++j) zero[j] = (__bf16)0.0f;
+  const int vtok = tid % LAC, vc = (tid / LAC) * 8;
+  auto fetch = [&](int c0) {
     const int cnt = min(LAC, n - c0);
     const bf16_t* base = proj + (int64_t)(t0 + c0) * ldp;
+    #pragma unroll
+    for (int i = 0; i < KI; ++i) {
+      const int tok = (i * 256 + tid) % LAC, c = (i * 256 + tid) / LAC * 8;
+      kraw[i] = zero;
+      if (tok < cnt && c < dk)
+        kraw[i] = *reinterpret_cast<const bf16v8*>(base + (int64_t)tok * ldp + nq + h * dk + c);
+    }
+    vraw = zero;
+    if (vtok < cnt && v0 + vc < vd)
+      vraw = *reinterpret_cast<const bf16v8*>(base + (int64_t)vtok * ldp + 2 * nq + h * vd + v0 + vc);
+    const int qi = wave * 16 + lrow;
+    #pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const int c = ks * 32 + lk * 8;
+      qraw[ks] = zero;
+      if (qi < cnt && c < dk)
+        qraw[ks] = *reinterpret_cast<const bf16v8*>(base + (int64_t)qi * ldp + h * dk + c);
+    }
+  };
+  fetch(0);
+
+  for (int c0 = 0; c0 < n; c0 += LAC) {
+    const int cnt = min(LAC, n - c0);
     __syncthreads();                               // the previous chunk's LDS reads are done
-    // keys, activated: token-major and key-major; zero past the chunk and past dk
-    for (int i = tid; i < LAC * (DP / 8); i += 256) {
-      const int tok = i % LAC, c = (i / LAC) * 8;
+    // keys, activated (silu(0) = 0: padding stays zero), token-major and key-major
+    #pragma unroll
+    for (int i = 0; i < KI; ++i) {
+      const int tok = (i * 256 + tid) % LAC, c = (i * 256 + tid) / LAC * 8;
       bf16v8 kv;
       #pragma unroll
-      for (int j = 0; j < 8; ++j) kv[j] = (__bf16)0.0f;
-      if (tok < cnt && c < dk) {
-        kv = *reinterpret_cast<const bf16v8*>(base + (int64_t)tok * ldp + nq + h * dk + c);
-        #pragma unroll
-        for (int j = 0; j < 8; ++j) kv[j] = (__bf16)la_silu((float)kv[j]);
-      }
+      for (int j = 0; j < 8; ++j) kv[j] = la_silu_bf16(kraw[i][j]);
       *reinterpret_cast<bf16v8*>(k_lds + tok * KPT + c) = kv;
       #pragma unroll
       for (int j = 0; j < 8; ++j) kT[(c + j) * LAC_TP + tok] = kv[j];
     }
     // values, activated, as they are and decayed to the chunk's end
     {
-      const int tok = tid % LAC, c = (tid / LAC) * 8;
-      bf16v8 vv;
-      #pragma unroll
-      for (int j = 0; j < 8; ++j) vv[j] = (__bf16)0.0f;
-      float dec = 0.f;
-      if (tok < cnt) {
-        dec = pw[cnt - 1 - tok];
-        if (v0 + c < vd) {
-          vv = *reinterpret_cast<const bf16v8*>(base + (int64_t)tok * ldp + 2 * nq + h * vd + v0 + c);
-          #pragma unroll
-          for (int j = 0; j < 8; ++j) vv[j] = (__bf16)la_silu((float)vv[j]);
-        }
-      }
+      const float dec = (vtok < cnt) ? pw[cnt - 1 - vtok] : 0.f;
       #pragma unroll
       for (int j = 0; j < 8; ++j) {
-        const int at = (c + j) * LAC_TP + tok;
-        vT[at] = vv[j];
+        const int at = (vc + j) * LAC_TP + vtok;
+        const __bf16 v = la_silu_bf16(vraw[j]);
+        vT[at] = v;
         __bf16 hi, lo;
-        la_split((float)vv[j] * dec, &hi, &lo);
+        la_split((float)v * dec, &hi, &lo);
         vh[at] = hi;
         vl[at] = lo;
       }
@@ -212,23 +232,13 @@ __global__ __launch_bounds__(256, 2) void linear_attention_chunk_kernel(
         }
       }
     }
-    // the wave's queries, activated, as A fragments
     bf16v8 qf[KS];
-    {
-      const int qi = wave * 16 + lrow;
+    #pragma unroll
+    for (int ks = 0; ks < KS; ++ks)
       #pragma unroll
-      for (int ks = 0; ks < KS; ++ks) {
-        #pragma unroll
-        for (int j = 0; j < 8; ++j) qf[ks][j] = (__bf16)0.0f;
-        const int c = ks * 32 + lk * 8;
-        if (qi < cnt && c < dk) {
-          qf[ks] = *reinterpret_cast<const bf16v8*>(base + (int64_t)qi * ldp + h * dk + c);
-          #pragma unroll
-          for (int j = 0; j < 8; ++j) qf[ks][j] = (__bf16)la_silu((float)qf[ks][j]);
-        }
-      }
-    }
+      for (int j = 0; j < 8; ++j) qf[ks][j] = la_silu_bf16(qraw[ks][j]);
     __syncthreads();
+    if (c0 + LAC < n) fetch(c0 + LAC);             // lands while this chunk is computed
     if (wave * 16 < cnt) {
       // what the state before the chunk gives
       f32x4 acc[2];

@@ -7,7 +7,7 @@
 //   out = S gelu_tanh(y)
 // Kernels:
 //   linear_unit_tile   bf16 prompt steps, one workgroup per (tile of <= 64
-//                      tokens of a sequence, block, 64 channels): convolution
+//                      tokens of a sequence, block, 64 or 128 channels): convolution
 //                      into LDS, both gates on MFMA (u as two bf16 terms, hi +
 //                      lo), then the recurrence inside the tile as prefixes
 //                      (P_t, Q_t): S_t = P_t S_start + Q_t
@@ -45,6 +45,29 @@ SM_INLINE void lu_gate(const lu_args& A, int ch, float zr, float zi, float u, fl
   const float la = -A.c * r * lu_softplus(A.lam[ch]);
   *a = expf(la);
   *b = sqrtf(-expm1f(2.0f * la)) * i * u;
+}
+
+// The same for the bf16 kernels on the hardware's exponential, reciprocal and
+// square root, with what depends on the channel only (biases, c softplus(lam))
+// taken once: errors of a few fp32 roundings. 1 - a^2 = -expm1(2 log a) by its
+// series where the exponential would cancel.
+struct lu_channel { float br, bi, csp; };
+SM_INLINE lu_channel lu_channel_of(const lu_args& A, int ch) {
+  return {A.gates_b[ch], A.gates_b[A.W + ch], A.c * lu_softplus(A.lam[ch])};
+}
+SM_INLINE void lu_gate_fast(const lu_channel& C, float zr, float zi, float u, float* a, float* b) {
+  const float la = -C.csp * sm_fast_sigmoid(zr + C.br);
+  const float e = 2.0f * la;
+  float p = fmaf(e, 1.0f / 7.0f, 1.0f);
+  p = fmaf(e * (1.0f / 6.0f), p, 1.0f);
+  p = fmaf(e * (1.0f / 5.0f), p, 1.0f);
+  p = fmaf(e * (1.0f / 4.0f), p, 1.0f);
+  p = fmaf(e * (1.0f / 3.0f), p, 1.0f);
+  p = fmaf(e * (1.0f / 2.0f), p, 1.0f);
+  const float x = __expf(la);
+  const float left = (e > -0.25f) ? -e * p : fmaf(-x, x, 1.0f);
+  *a = x;
+  *b = __builtin_amdgcn_sqrtf(left) * sm_fast_sigmoid(zi + C.bi) * u;
 }
 
 // u of channel ch for the token whose x row starts at xr, rel tokens into its
@@ -100,17 +123,20 @@ SM_INLINE void lu_split(const float* u, bf16v8* hi, bf16v8* lo) {
 // ---- prompt tiles
 #define LUT_KC 128            // channels of a block staged at once
 #define LUT_KP (LUT_KC + 8)
-template <int TAPS>
-__global__ __launch_bounds__(256, 2) void linear_unit_tile_kernel(
+// NW waves, 16 channels each: with 8 the block's convolution is redone half as
+// often.
+template <int TAPS, int NW>
+__global__ __launch_bounds__(64 * NW, 2) void linear_unit_tile_kernel(
     const bf16_t* __restrict__ x,         // x part of the projection rows
     const bf16_t* __restrict__ gw,        // [2, blocks, n, n]
     const int* __restrict__ tiles,        // [ntiles, 3] = (row, first token, tokens)
     lu_args A, float* __restrict__ P, float* __restrict__ Q) {
   __shared__ __attribute__((aligned(16))) __bf16 uh[64 * LUT_KP];
   __shared__ __attribute__((aligned(16))) __bf16 ul[64 * LUT_KP];
-  __shared__ float own[64][65];           // fp32 u of the workgroup's own channels
+  constexpr int NC = 16 * NW;
+  __shared__ float own[64][NC + 1];       // fp32 u of the workgroup's own channels
   const int b = tiles[3 * blockIdx.x], t0 = tiles[3 * blockIdx.x + 1], nt = tiles[3 * blockIdx.x + 2];
-  const int blk = blockIdx.y, c0 = blockIdx.z * 64, n = A.n;
+  const int blk = blockIdx.y, c0 = blockIdx.z * NC, n = A.n;
   const int tid = threadIdx.x, wave = tid >> 6, l = tid & 63, lrow = l & 15, lk = l >> 4;
   const int rel0 = t0 - A.cu[b];
   const float* tl = A.tails + (int64_t)A.slots[b] * (A.taps - 1) * A.W;
@@ -124,7 +150,7 @@ __global__ __launch_bounds__(256, 2) void linear_unit_tile_kernel(
     for (int mt = 0; mt < 4; ++mt) acc[g][mt] = f32x4{0.f, 0.f, 0.f, 0.f};
   for (int k0 = 0; k0 < n; k0 += LUT_KC) {
     __syncthreads();
-    // convolution: a thread takes 8 channels for 4 neighbouring tokens
+    // convolution: a thread takes 8 channels for a few neighbouring tokens
     {
       const int kc = (tid & 15) * 8, ch = blk * n + k0 + kc;
       const bool in = k0 + kc < n;
@@ -134,8 +160,8 @@ __global__ __launch_bounds__(256, 2) void linear_unit_tile_kernel(
         for (int e = 0; e < 8 * TAPS; ++e) wr[e] = A.conv_w[(int64_t)ch * TAPS + e];
       }
       #pragma unroll
-      for (int s = 0; s < 4; ++s) {
-        const int tok = (tid >> 4) * 4 + s;
+      for (int s = 0; s < 16 / NW; ++s) {
+        const int tok = (tid >> 4) * (16 / NW) + s;
         float u[8];
         #pragma unroll
         for (int e = 0; e < 8; ++e) u[e] = 0.f;
@@ -146,7 +172,7 @@ __global__ __launch_bounds__(256, 2) void linear_unit_tile_kernel(
         *reinterpret_cast<bf16v8*>(uh + tok * LUT_KP + kc) = hi;
         *reinterpret_cast<bf16v8*>(ul + tok * LUT_KP + kc) = lo;
         const int oc = k0 + kc - c0;
-        if (oc >= 0 && oc < 64) {
+        if (oc >= 0 && oc < NC) {
           #pragma unroll
           for (int e = 0; e < 8; ++e) own[tok][oc + e] = u[e];
         }
@@ -177,7 +203,7 @@ __global__ __launch_bounds__(256, 2) void linear_unit_tile_kernel(
     }
   }
   // prefixes: the lane's 4 tokens, then the 4 lane groups, then the 16-token tiles
-  const int ch = blk * n + min(col, n - 1);
+  const lu_channel C = lu_channel_of(A, blk * n + min(col, n - 1));
   float pt = 1.f, qt = 0.f;                          // everything before the 16-token tile
   #pragma unroll
   for (int mt = 0; mt < 4; ++mt) {
@@ -187,7 +213,7 @@ __global__ __launch_bounds__(256, 2) void linear_unit_tile_kernel(
       const int tok = mt * 16 + lk * 4 + r;
       float a = 1.f, bb = 0.f;
       if (tok < nt)
-        lu_gate(A, ch, acc[0][mt][r], acc[1][mt][r], own[tok][wave * 16 + lrow], &a, &bb);
+        lu_gate_fast(C, acc[0][mt][r], acc[1][mt][r], own[tok][wave * 16 + lrow], &a, &bb);
       p[r] = r ? a * p[r ? r - 1 : 0] : a;
       q[r] = r ? fmaf(a, q[r ? r - 1 : 0], bb) : bb;
     }
@@ -319,6 +345,7 @@ __global__ __launch_bounds__(256) void linear_unit_step_kernel(
   __syncthreads();
   if (wave > 0 || col >= n) return;
   const int ch = blk * n + col;
+  const lu_channel C = lu_channel_of(A, ch);
   #pragma unroll
   for (int r = 0; r < 4; ++r) {
     const int t = t0 + lk * 4 + r;
@@ -332,7 +359,7 @@ __global__ __launch_bounds__(256) void linear_unit_step_kernel(
     const int64_t slot = A.slots[t];
     const float u = lu_conv(A, x + (int64_t)t * A.ldp, 0, A.tails + slot * keep * A.W, ch);
     float a, b;
-    lu_gate(A, ch, zr, zi, u, &a, &b);
+    lu_gate_fast(C, zr, zi, u, &a, &b);
     float* st = state + slot * A.W + ch;
     const float S = fmaf(a, *st, b);
     *st = S;
@@ -454,13 +481,12 @@ torch::Tensor linear_unit(torch::Tensor proj, torch::Tensor conv_w, torch::Tenso
       const int* tp = tiles->data_ptr<int>();
       auto P = torch::empty({T, (int64_t)W}, f32), Q = torch::empty({T, (int64_t)W}, f32);
       auto S0 = torch::empty({nt, (int64_t)W}, f32);
-      const dim3 grid(nt, blocks, SM_CDIV(n, 64));
-      if (taps == 4)
-        linear_unit_tile_kernel<4><<<grid, 256, 0, stream>>>(xp, gp, tp, A, P.data_ptr<float>(),
-                                                             Q.data_ptr<float>());
-      else
-        linear_unit_tile_kernel<0><<<grid, 256, 0, stream>>>(xp, gp, tp, A, P.data_ptr<float>(),
-                                                             Q.data_ptr<float>());
+#define LU_TILE(TAPS, NW)                                                              \
+  linear_unit_tile_kernel<TAPS, NW><<<dim3(nt, blocks, SM_CDIV(n, 16 * NW)), 64 * NW, 0, stream>>>( \
+      xp, gp, tp, A, P.data_ptr<float>(), Q.data_ptr<float>())
+      if (n <= 64) { if (taps == 4) LU_TILE(4, 4); else LU_TILE(0, 4); }
+      else { if (taps == 4) LU_TILE(4, 8); else LU_TILE(0, 8); }
+#undef LU_TILE
       SM_CHECK_LAUNCH();
       linear_unit_carry_kernel<<<dim3(B, SM_CDIV(W, 64)), 64, 0, stream>>>(
           P.data_ptr<float>(), Q.data_ptr<float>(), tp, tile_cu->data_ptr<int>(), A.slots, W, sp,

@@ -37,9 +37,9 @@ typedef __attribute__((ext_vector_type(4))) float f32x4;
 namespace {
 
 // cap tanh(x / cap), tanh z = 1 - 2 / (1 + e^(2z)): absolute error of a few
-// fp32 roundings of cap; saturates to +-cap.
-SM_INLINE float wam_cap(float x, float cap, float icap) {
-  return cap - 2.0f * cap / (1.0f + __expf(2.0f * x * icap));
+// fp32 roundings of cap; saturates to +-cap. ic2 = 2 / cap.
+SM_INLINE float wam_cap(float x, float cap, float ic2) {
+  return fmaf(-2.0f * cap, __builtin_amdgcn_rcpf(1.0f + __expf(x * ic2)), cap);
 }
 
 // NT: 16-column value tiles per wave (vd <= 16 NT); KS: 32-entry steps of the
@@ -87,7 +87,7 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
   float* p_lds = p_all + wave * 16 * WAM_PP;
   float* tb = tb_all + wave * WAM_TB;
   const bool active = wave * 16 < nq;
-  const float icap = CAP ? 1.0f / vw.cap : 0.f;
+  const float ic2 = CAP ? 2.0f / vw.cap : 0.f;
   const float a1 = DIST ? r1[hd] : 0.f, a2 = DIST ? r2[hd] : 0.f;
 
   // the wave's queries as A fragments: row lrow, k = ks * 32 + lk * 8 ..
@@ -205,7 +205,7 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
           const int j = (i < nf) ? i : lo + (i - nf);
           const bool seen = i < n && j <= prow && (j >= first[r] || j < vw.keep);
           float x = s[ct][r] * scale;
-          if (CAP) x = wam_cap(x, vw.cap, icap);
+          if (CAP) x = wam_cap(x, vw.cap, ic2);
           if (DIST) {
             if (tabled) x -= tb[lk * 4 + r + (KB - 1) - (ct * 16 + lrow)];
             else if (seen) x -= a1 * log1pf(a2 * (float)(prow - j));

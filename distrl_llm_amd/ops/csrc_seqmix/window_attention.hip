@@ -902,7 +902,7 @@ torch::Tensor qk_prepare_kv_write(torch::Tensor proj, int64_t heads, int64_t kv_
 }
 
 // defined in window_attention_mfma.hip
-bool window_attention_mfma_fits(int KD, int vd, int maps, bool dist, bool cap);
+bool window_attention_mfma_fits(int KD, int vd, int maps, bool dist, bool ext);
 void window_attention_mfma(torch::Tensor q, int KD, torch::Tensor cache, int H, int G, int dk, int vd,
                            int whole_key, torch::Tensor block_tables, int block_size,
                            torch::Tensor positions, float scale, wa_view vw,
@@ -978,7 +978,7 @@ torch::Tensor window_attention(torch::Tensor q, torch::Tensor cache, int64_t hea
   const bool is_bf16 = q.scalar_type() == at::kBFloat16;
   if (!is_bf16) SM_CHECK_F32(q);
   if (is_bf16 && tiles.has_value() && max_tile_queries > 4 &&
-      window_attention_mfma_fits(KD, vd, MP, r1.has_value(), softcap > 0.0)) {
+      window_attention_mfma_fits(KD, vd, MP, r1.has_value(), softcap > 0.0 || chunk > 0)) {
     SM_CHECK_CUDA(*tiles); SM_CHECK_I32(*tiles);
     TORCH_CHECK(tiles->dim() == 2 && tiles->size(1) == 3 && max_tile_queries <= 64,
                 "window_attention: tiles");

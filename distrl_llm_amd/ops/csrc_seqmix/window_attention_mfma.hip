@@ -45,8 +45,9 @@ SM_INLINE float wam_cap(float x, float cap, float ic2) {
 // NT: 16-column value tiles per wave (vd <= 16 NT); KS: 32-entry steps of the
 // query/key dot product held in registers (KD <= 32 KS); KB: keys per block;
 // DIST: the distance bias is taken off the scores (r1, r2 given); MAPS: query
-// and key maps per head; CAP: scores become cap tanh(score / cap).
-template <int NT, int KS, int KB, bool DIST, int MAPS, bool CAP>
+// and key maps per head; EXT: chunks and capped scores (without it the view is a
+// window at most, which costs the register-bound variants nothing).
+template <int NT, int KS, int KB, bool DIST, int MAPS, bool EXT>
 __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
     const bf16_t* __restrict__ q, int KD,  // [Tn, H MAPS, KD]
     const bf16_t* __restrict__ cache,      // [rows, G (MAPS dk + vd)]
@@ -87,7 +88,7 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
   float* p_lds = p_all + wave * 16 * WAM_PP;
   float* tb = tb_all + wave * WAM_TB;
   const bool active = wave * 16 < nq;
-  const float ic2 = CAP ? 2.0f / vw.cap : 0.f;
+  const float ic2 = (EXT && vw.cap > 0.f) ? 2.0f / vw.cap : 0.f;
   const float a1 = DIST ? r1[hd] : 0.f, a2 = DIST ? r2[hd] : 0.f;
 
   // the wave's queries as A fragments: row lrow, k = ks * 32 + lk * 8 ..
@@ -107,9 +108,10 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
   // padding rows of v_lds (value columns vd .. NVp) stay zero
   for (int i = tid; i < (NVp - vd) * WAM_VP; i += 256) v_lds[vd * WAM_VP + i] = __float2bfloat16(0.f);
 
-  int first[4];                                    // where each of the lane's queries starts to see
+  int first[EXT ? 4 : 1];                          // where each of the lane's queries starts to see
   #pragma unroll
-  for (int r = 0; r < 4; ++r) first[r] = wa_first(vw, p0 + min(wave * 16 + lk * 4 + r, nq - 1));
+  for (int r = 0; r < 4 && EXT; ++r)
+    first[r] = wa_first(vw, p0 + min(wave * 16 + lk * 4 + r, nq - 1));
   float m[MAPS][4], lsum[MAPS][4];
   f32x4 acc[MAPS][NT];
   #pragma unroll
@@ -160,7 +162,11 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
       const int jb0 = lo + (i0 - nf);
       const int wq_last = min(plast, p0 + wave * 16 + 15), wq_first = p0 + wave * 16;
       if (jb0 > wq_last) continue;
-      if (jb0 + WAM_KB - 1 < wa_first(vw, wq_first) && jb0 >= vw.keep) continue;
+      if (EXT) {
+        if (jb0 + WAM_KB - 1 < wa_first(vw, wq_first) && jb0 >= vw.keep) continue;
+      } else if (vw.window > 0 && jb0 + WAM_KB - 1 < wq_first - vw.window + 1 && jb0 >= vw.keep) {
+        continue;
+      }
     }
 
     // distance bias of this wave and block: the block's keys are consecutive
@@ -203,9 +209,10 @@ __global__ __launch_bounds__(256, 2) void window_attention_mfma_kernel(
         for (int ct = 0; ct < KB / 16; ++ct) {
           const int i = i0 + ct * 16 + lrow;
           const int j = (i < nf) ? i : lo + (i - nf);
-          const bool seen = i < n && j <= prow && (j >= first[r] || j < vw.keep);
+          const bool in = EXT ? j >= first[EXT ? r : 0] : vw.window <= 0 || prow - j < vw.window;
+          const bool seen = i < n && j <= prow && (in || j < vw.keep);
           float x = s[ct][r] * scale;
-          if (CAP) x = wam_cap(x, vw.cap, ic2);
+          if (EXT) x = (ic2 > 0.f) ? wam_cap(x, vw.cap, ic2) : x;
           if (DIST) {
             if (tabled) x -= tb[lk * 4 + r + (KB - 1) - (ct * 16 + lrow)];
             else if (seen) x -= a1 * log1pf(a2 * (float)(prow - j));
@@ -313,8 +320,8 @@ size_t wam_lds_bytes(int KD, int vd, bool dist, int maps) {
 
 // 16-byte pieces of the cache rows: the key columns a head meets (dim, or
 // kv_heads * dim for folded queries) and the value size are multiples of 8
-bool window_attention_mfma_fits(int KD, int vd, int maps, bool dist, bool cap) {
-  return !(cap && (dist || maps == 2)) && KD % 8 == 0 && vd % 8 == 0 &&
+bool window_attention_mfma_fits(int KD, int vd, int maps, bool dist, bool ext) {
+  return !(ext && (dist || maps == 2)) && KD % 8 == 0 && vd % 8 == 0 &&
          KD <= (maps == 2 ? 128 : 512) && vd <= 256 &&
          wam_lds_bytes(KD, vd, true, maps) <= 150 * 1024;
 }
@@ -329,9 +336,9 @@ void window_attention_mfma(torch::Tensor q, int KD, torch::Tensor cache, int H, 
   auto stream = at::cuda::getCurrentCUDAStream();
   const size_t lds = wam_lds_bytes(KD, vd, r1 != nullptr, maps);
   dim3 grid(ntiles, H);
-#define WAM_LAUNCH(NT, KS, DIST, MAPS, CAP)                                                       \
+#define WAM_LAUNCH(NT, KS, DIST, MAPS, EXT)                                                    \
   do {                                                                                         \
-    auto kern = window_attention_mfma_kernel<NT, KS, WAM_KEYS, DIST, MAPS, CAP>;                  \
+    auto kern = window_attention_mfma_kernel<NT, KS, WAM_KEYS, DIST, MAPS, EXT>;                  \
     static int raised = 0;                                                                     \
     if (lds > 64 * 1024 && (int)lds > raised) {                                                \
       TORCH_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(kern),                     \
@@ -347,11 +354,11 @@ void window_attention_mfma(torch::Tensor q, int KD, torch::Tensor cache, int H, 
         reinterpret_cast<const bf16_t*>(gate), ldg, gs, df,                                    \
         reinterpret_cast<bf16_t*>(out.data_ptr()));                                            \
   } while (0)
-#define WAM_BY_KS(NT, DIST, CAP)                             \
+#define WAM_BY_KS(NT, DIST, EXT)                             \
   do {                                                       \
-    if (KD <= 128) WAM_LAUNCH(NT, 4, DIST, 1, CAP);          \
-    else if (KD <= 256) WAM_LAUNCH(NT, 8, DIST, 1, CAP);     \
-    else WAM_LAUNCH(NT, 16, DIST, 1, CAP);                   \
+    if (KD <= 128) WAM_LAUNCH(NT, 4, DIST, 1, EXT);          \
+    else if (KD <= 256) WAM_LAUNCH(NT, 8, DIST, 1, EXT);     \
+    else WAM_LAUNCH(NT, 16, DIST, 1, EXT);                   \
   } while (0)
 #define WAM_BY_KS2(NT)                                       \
   do {                                                       \
@@ -364,11 +371,11 @@ void window_attention_mfma(torch::Tensor q, int KD, torch::Tensor cache, int H, 
     else if (vd <= 128) BY(8, ##__VA_ARGS__);                \
     else BY(16, ##__VA_ARGS__);                              \
   } while (0)
-  // capped scores: one map without distance bias (the caller sends the rest of
-  // the combinations to the other kernels)
+  // chunks and capped scores: one map without distance bias (the caller sends
+  // the rest of the combinations to the other kernels)
   if (maps == 2) WAM_BY_NT(WAM_BY_KS2);
   else if (r1 != nullptr) WAM_BY_NT(WAM_BY_KS, true, false);
-  else if (vw.cap > 0.f) WAM_BY_NT(WAM_BY_KS, false, true);
+  else if (vw.cap > 0.f || vw.chunk > 0) WAM_BY_NT(WAM_BY_KS, false, true);
   else WAM_BY_NT(WAM_BY_KS, false, false);
 #undef WAM_BY_NT
 #undef WAM_BY_KS2

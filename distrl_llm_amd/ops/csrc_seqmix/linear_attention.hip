@@ -105,7 +105,8 @@ __global__ __launch_bounds__(256) void linear_attention_scan_kernel(
 
 // ---- chunks of 64 tokens. One workgroup (4 waves) per (row, head, 32 value
 // columns); wave w owns the queries 16 w .. of a chunk and the 16-key tiles w,
-// w + 4, ... of the state. KS: 32-entry steps of the key axis (dk <= 32 KS).
+// w + 4, ... of the state. Rows are the slowest grid axis: rows of a few tokens
+// beside long ones then leave the chip evenly filled. KS: 32-entry steps of the key axis (dk <= 32 KS).
 // MFMA 16x16x32 bf16 fragments: A lane l -> row l & 15, k (l >> 4) * 8 ..;
 // B lane l -> column l & 15, same k; D lane l reg r -> row (l >> 4) * 4 + r,
 // column l & 15.
@@ -138,7 +139,7 @@ __global__ __launch_bounds__(256, 2) void linear_attention_chunk_kernel(
   __bf16* sl = sh + LAC_V * KPT;
   float* p_all = reinterpret_cast<float*>(sl + LAC_V * KPT);      // [4][16][LAC_PP]
   float* pw = p_all + 4 * 16 * LAC_PP;                            // [LAC + 1] powers of the decay
-  const int b = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * LAC_V;
+  const int h = blockIdx.x, v0 = blockIdx.y * LAC_V, b = blockIdx.z;
   const int tid = threadIdx.x, wave = tid >> 6, l = tid & 63, lrow = l & 15, lk = l >> 4;
   const int t0 = cu[b], n = cu[b + 1] - t0;
   if (n == 0) return;
@@ -392,6 +393,7 @@ torch::Tensor linear_attention(torch::Tensor proj, int64_t heads, int64_t dim, i
   const int64_t T = proj.size(0);
   const int H = heads, dk = dim, vd = vdim, B = slots.numel();
   const int nq = H * dk, nv = H * vd;
+  TORCH_CHECK(B <= 65535, "linear_attention: more than 65535 rows in a step");
   TORCH_CHECK(H >= 1 && dk >= 1 && vd >= 1 && dk <= 512, "linear_attention: key size above 512");
   TORCH_CHECK(proj.is_cuda() && proj.dim() == 2 && proj.stride(1) == 1 &&
               proj.size(1) >= 2 * (int64_t)nq + 2 * nv, "linear_attention: rows are [q | k | v | gate]");
@@ -418,7 +420,7 @@ torch::Tensor linear_attention(torch::Tensor proj, int64_t heads, int64_t dim, i
                        ldp % 8 == 0 && reinterpret_cast<uintptr_t>(proj.data_ptr()) % 16 == 0;
   if (chunked) {
     const bf16_t* xp = reinterpret_cast<const bf16_t*>(proj.data_ptr());
-    const dim3 grid(B, H, SM_CDIV(vd, LAC_V));
+    const dim3 grid(H, SM_CDIV(vd, LAC_V), B);
     if (dk <= 64) launch_chunk<2>(grid, stream, xp, ldp, H, dk, vd, pp, np, sp, cp, sl, op);
     else if (dk <= 128) launch_chunk<4>(grid, stream, xp, ldp, H, dk, vd, pp, np, sp, cp, sl, op);
     else launch_chunk<8>(grid, stream, xp, ldp, H, dk, vd, pp, np, sp, cp, sl, op);

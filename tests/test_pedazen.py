@@ -241,7 +241,7 @@ def test_linear_unit_op(dev, W, blocks, taps):
             assert rel_err(tails[2 - 2 * b, k], x[lengths[b] - taps + 1 + k, W:]) < 1e-6
 
 
-@pytest.mark.parametrize("E,top,groups", [(12, 4, (4, 3)), (6, 2, (3, 1)), (6, 3, (2, 1)),
+@pytest.mark.parametrize("E,top,groups", [(15, 4, (5, 3)), (6, 2, (3, 1)), (6, 3, (2, 1)),
                                           (5, 3, None), (8, 8, (4, 4)), (9, 2, (9, 2)), (1, 1, None),
                                           (64, 6, (8, 3))])
 def test_router_and_experts(dev, E, top, groups):
